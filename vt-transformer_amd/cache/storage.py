@@ -12,7 +12,7 @@ a NaN into a weighted sum.
 """
 from __future__ import annotations
 
-from dataclasses import dataclass
+from dataclasses import dataclass, replace
 from typing import Dict, List, Optional
 
 import torch
@@ -89,6 +89,13 @@ class CacheStorage:
                 if need is None or src is None or not need.same_layout(src):
                     raise ValueError(f"schedule entry {i} cannot read the cache of entry {e.cache_from}: "
                                      f"their pages differ")
+        # A cache that further entries read keeps a token until the last of its readers has passed it: an entry's need
+        # has the widest window among its own and its readers' (0 if one of them sees every token).
+        for i, e in enumerate(schedule):
+            if e.cache_from is not None:
+                own, reach = needs[e.cache_from], needs[i].window
+                keep = max(own.window, reach) if own.window > 0 and reach > 0 else 0
+                needs[e.cache_from] = replace(own, window=keep)
         # groups of entries with their own cache and equal needs
         keys: List = []
         self.group_needs: List[CacheNeed] = []

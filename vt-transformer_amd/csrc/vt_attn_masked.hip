@@ -20,6 +20,9 @@
 //                   and mixes values across layers: vmix 1 leaves the token's values in `v_first` (float32), vmix 2
 //                   writes (1 - lambda) v + lambda v_first into the pages instead of v.  With `q_gain` / `k_gain`
 //                   ([D], shared by the heads) the unit-RMS queries / keys are multiplied by a gain per element.
+//   vt_qk_prepare_whole: the same step for a mixer that norms queries and keys over the whole projection: all H D
+//                   query elements of a token divided by their common root mean square and multiplied by a gain per
+//                   element ([H D]), the G D key elements likewise by theirs; no rotation.
 //   vt_attn_masked, further forms of the score and of the weights, each switched on by its pointer or flag:
 //                   `dist_r1`, `dist_r2` ([H] each): r1[head] * ln(1 + r2[head] * (i - j)) is taken off the score;
 //                   `score_shift` ([H]): a number per head is added to every score;
@@ -178,6 +181,124 @@ extern "C" int vt_qk_prepare(const void* x, int x_dtype, long long ldx, const fl
     else if (x_dtype == VT_BF16 && cache_dtype == VT_BF16) qk_prepare_kernel<bf16_t, bf16_t><<<grid, 256, 0, stream>>>(a);
     else return vt_fail("vt_qk_prepare: dtypes %d -> %d are not handled", x_dtype, cache_dtype);
     VT_CHECK_LAUNCH("vt_qk_prepare");
+    return 0;
+}
+
+// ---------------------------------------------------------------------------
+// Queries and keys normed over the whole projection.  Per token one block for the queries, one for the keys and one for
+// the values; a row's sum of squares is taken in an order that depends on its length alone.
+// ---------------------------------------------------------------------------
+struct WholeArgs {
+    const void* x;          // [n][ldx]: H D query elements, then (write_kv) G D key and G Dv value elements
+    const int* positions;
+    const int* tok_entry;
+    const int* block_table;
+    void* q_out;            // [n][H D]
+    void* k_pages;          // [page][G][slot][D]
+    void* v_pages;          // [page][G][Dv][slot]
+    const float* q_gain;    // [H D]
+    const float* k_gain;    // [G D]
+    long long ldx;
+    int H, G, D, Dv, page_size, max_blocks, num_pages;
+    float eps;
+};
+
+__device__ __forceinline__ float4 whole_load4(const float* p) { return *(const float4*)p; }
+__device__ __forceinline__ float4 whole_load4(const bf16_t* p) {
+    const uint2 u = *(const uint2*)p;
+    return make_float4(lowp_lo(u.x), lowp_hi(u.x), lowp_lo(u.y), lowp_hi(u.y));
+}
+__device__ __forceinline__ void whole_store4(float* p, float4 v) { *(float4*)p = v; }
+__device__ __forceinline__ void whole_store4(bf16_t* p, float4 v) {
+    uint2 u;
+    u.x = vt_pack2(v.x, v.y);
+    u.y = vt_pack2(v.z, v.w);
+    *(uint2*)p = u;
+}
+
+// VEC: head sizes and the row's length are multiples of 4 (a piece of four elements lies in one head)
+template <typename TI, typename TC, bool VEC>
+__global__ __launch_bounds__(256) void qk_prepare_whole_kernel(WholeArgs a) {
+    __shared__ float red[16];
+    const int t = blockIdx.x, part = blockIdx.y, tid = threadIdx.x;
+    const TI* x = (const TI*)a.x + (size_t)t * a.ldx;
+    int pg = 0, slot = 0;
+    if (part > 0) {
+        const int pos = a.positions[t];
+        const int blk = pos / a.page_size;
+        pg = blk < a.max_blocks ? a.block_table[(size_t)a.tok_entry[t] * a.max_blocks + blk] : -1;
+        if (pg < 0 || pg >= a.num_pages) return;        // (a padding entry of a recorded step has no page)
+        slot = pos - blk * a.page_size;
+    }
+    if (part == 2) {
+        const TI* v = x + (size_t)(a.H + a.G) * a.D;
+        TC* dst = (TC*)a.v_pages + (size_t)pg * a.G * a.Dv * a.page_size + slot;
+        for (int i = tid; i < a.G * a.Dv; i += 256) store_f32<TC>(dst, (size_t)i * a.page_size, load_f32<TI>(v, i));
+        return;
+    }
+    const int len = (part == 0 ? a.H : a.G) * a.D;
+    const TI* src = part == 0 ? x : x + (size_t)a.H * a.D;
+    const float* gain = part == 0 ? a.q_gain : a.k_gain;
+    float ss = 0.f;
+    if constexpr (VEC) {
+        for (int i = tid * 4; i < len; i += 1024) {
+            const float4 v = whole_load4(src + i);
+            ss = fmaf(v.x, v.x, fmaf(v.y, v.y, fmaf(v.z, v.z, fmaf(v.w, v.w, ss))));
+        }
+    } else {
+        for (int i = tid; i < len; i += 256) {
+            const float v = load_f32<TI>(src, i);
+            ss = fmaf(v, v, ss);
+        }
+    }
+    ss = block_sum(ss, red);
+    const float r = 1.0f / sqrtf(ss / (float)len + a.eps);
+    TC* q = (TC*)a.q_out + (size_t)t * a.H * a.D;
+    TC* k = (TC*)a.k_pages + ((size_t)pg * a.G * a.page_size + slot) * a.D;
+    // element i of the keys: head i / D's row of this slot
+    auto place = [&](int i) -> TC* {
+        if (part == 0) return q + i;
+        const int g = i / a.D;
+        return k + (size_t)g * a.page_size * a.D + (i - g * a.D);
+    };
+    if constexpr (VEC) {
+        for (int i = tid * 4; i < len; i += 1024) {
+            const float4 v = whole_load4(src + i), g = *(const float4*)(gain + i);
+            whole_store4(place(i), make_float4(v.x * r * g.x, v.y * r * g.y, v.z * r * g.z, v.w * r * g.w));
+        }
+    } else {
+        for (int i = tid; i < len; i += 256) store_f32<TC>(place(i), 0, load_f32<TI>(src, i) * r * gain[i]);
+    }
+}
+
+extern "C" int vt_qk_prepare_whole(const void* x, int x_dtype, long long ldx, const int* positions, const int* tok_entry,
+                                   const int* block_table, int max_blocks, void* q_out, void* k_pages, void* v_pages,
+                                   int cache_dtype, int page_size, int num_pages, int n, int H, int G, int D, int Dv,
+                                   int write_kv, float eps, const float* q_gain, const float* k_gain, hipStream_t stream) {
+    VT_REQUIRE(n >= 0 && H > 0 && G > 0 && H % G == 0 && D > 0 && Dv > 0, "vt_qk_prepare_whole: bad heads %d/%d of %d/%d", H, G, D, Dv);
+    VT_REQUIRE((long long)H * D < (1ll << 30) && (long long)G * Dv < (1ll << 30), "vt_qk_prepare_whole: rows are too long");
+    VT_REQUIRE(ldx >= (long long)(H + (write_kv ? G : 0)) * D + (write_kv ? (long long)G * Dv : 0),
+               "vt_qk_prepare_whole: rows of %lld elements are too short", ldx);
+    VT_REQUIRE(!write_kv || (page_size > 0 && max_blocks > 0 && num_pages > 0 && positions && tok_entry && block_table && k_pages &&
+                             v_pages && k_gain), "vt_qk_prepare_whole: bad cache sizes");
+    VT_REQUIRE(q_gain != nullptr, "vt_qk_prepare_whole: no gains");
+    if (n == 0) return 0;
+    WholeArgs a;
+    a.x = x; a.positions = positions; a.tok_entry = tok_entry; a.block_table = block_table; a.q_out = q_out; a.k_pages = k_pages;
+    a.v_pages = v_pages; a.q_gain = q_gain; a.k_gain = k_gain; a.ldx = ldx; a.H = H; a.G = G; a.D = D; a.Dv = Dv;
+    a.page_size = page_size; a.max_blocks = max_blocks; a.num_pages = num_pages; a.eps = eps;
+    const bool vec = D % 4 == 0 && ldx % 4 == 0 && !(((uintptr_t)x | (uintptr_t)q_out | (uintptr_t)k_pages | (uintptr_t)q_gain |
+                                                      (uintptr_t)k_gain) & 15);
+    const dim3 grid(n, write_kv ? 3 : 1);
+#define VT_WHOLE(TI, TC) do { \
+        if (vec) qk_prepare_whole_kernel<TI, TC, true><<<grid, 256, 0, stream>>>(a); \
+        else qk_prepare_whole_kernel<TI, TC, false><<<grid, 256, 0, stream>>>(a); } while (0)
+    if (x_dtype == VT_F32 && cache_dtype == VT_F32) VT_WHOLE(float, float);
+    else if (x_dtype == VT_F32 && cache_dtype == VT_BF16) VT_WHOLE(float, bf16_t);
+    else if (x_dtype == VT_BF16 && cache_dtype == VT_BF16) VT_WHOLE(bf16_t, bf16_t);
+    else return vt_fail("vt_qk_prepare_whole: dtypes %d -> %d are not handled", x_dtype, cache_dtype);
+#undef VT_WHOLE
+    VT_CHECK_LAUNCH("vt_qk_prepare_whole");
     return 0;
 }
 

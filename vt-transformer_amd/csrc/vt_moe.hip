@@ -2,12 +2,18 @@
 //
 //   vt_moe_route:    logits z = W_r x in float32 (W_r is kept in float32), scores sigmoid(z) or softmax(z), the `top`
 //                    largest per token (the lower index among equals), optionally divided by their sum.  A block per token.
+//                    Further forms of the choice, each switched on by its pointer or number: `correction` [E] is added to
+//                    the scores for the choice only; the E outputs form `groups` runs of neighbours, of which only the
+//                    `keep` with the largest choice score in them are eligible; the last `identity` outputs are no
+//                    experts: a chosen one gets the id -1 and adds its weight to id_wts[token]; the weights are times
+//                    out_scale.
 //   vt_moe_gate_up:  for every (token, choice): act = f(W_gate,e xe) * (W_up,e xe), where xe is the token's input times
 //                    in_scale (the choice's score where the score multiplies the expert's input, else 1), rounded to the
 //                    runtime's type as an expert's input is; f(g) = g sigmoid(alpha g (1 + cubic g^2)).
 //   vt_moe_down:     out[t] = sum over the token's choices, in their order, of out_scale * W_down,e act.
 // These two read an expert's matrices once per token that chose it: the arrangement for few tokens, where every chosen
 // expert's matrices have to be read anyway.  (Many tokens go through vt_moe_sort and the grouped products below.)
+// A pair whose id is negative has no expert: no product is made for it and nothing of it is written or read.
 // Every sum is taken in an order that depends on the sizes alone, so a token's result does not depend on its batch.
 #include "vt_common.h"
 #include <math.h>
@@ -32,26 +38,38 @@ __device__ __forceinline__ float wave_dot_f32(const float* __restrict__ row, con
     return wave_sum(acc);
 }
 
+struct RouteArgs {
+    const void* x;              // [n][W]
+    const float* wr;            // [E][W]
+    const float* correction;    // [E] or null
+    int* ids;                   // [n][top]
+    float* wts;                 // [n][top]
+    float* id_wts;              // [n] or null: the weight of the chosen outputs that are no experts
+    int E, W, top, softmax, renorm, groups, keep, identity;
+    float renorm_eps, out_scale;
+};
+
 // A block of four waves per token: the token lies in LDS as float32, the waves take the experts in turn, and the
 // first wave then picks the largest scores.
 template <typename TI>
-__global__ __launch_bounds__(256) void moe_route_kernel(const TI* __restrict__ x, const float* __restrict__ wr,
-                                                        int* __restrict__ ids, float* __restrict__ wts, int E, int W, int top,
-                                                        int softmax, int renorm) {
-    extern __shared__ float sh[];       // W values of the token, then E scores
+__global__ __launch_bounds__(256) void moe_route_kernel(RouteArgs a) {
+    extern __shared__ float sh[];       // W values of the token, E scores, E choice scores, the groups' best
+    const int E = a.E, W = a.W, top = a.top;
     float* xs = sh;
     float* sc = sh + W;
+    float* ch = a.correction || a.groups > 1 ? sc + E : sc;     // (without either, the scores themselves are chosen from)
+    float* gb = sc + 2 * E;
     const int t = blockIdx.x, wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
-    const TI* xt = x + (size_t)t * W;
+    const TI* xt = (const TI*)a.x + (size_t)t * W;
     for (int j = threadIdx.x; j < W; j += 256) xs[j] = load_f32<TI>(xt, j);
     __syncthreads();
     for (int e = wave; e < E; e += 4) {
-        const float acc = wave_dot_f32(wr + (size_t)e * W, xs, W, lane);
+        const float acc = wave_dot_f32(a.wr + (size_t)e * W, xs, W, lane);
         if (lane == 0) sc[e] = acc;
     }
     __syncthreads();
     if (wave != 0) return;
-    if (softmax) {
+    if (a.softmax) {
         float m = -INFINITY;
         for (int e = lane; e < E; e += 64) m = fmaxf(m, sc[e]);
         m = wave_max(m);
@@ -64,12 +82,33 @@ __global__ __launch_bounds__(256) void moe_route_kernel(const TI* __restrict__ x
         for (int e = lane; e < E; e += 64) sc[e] = 1.0f / (1.0f + expf(-sc[e]));
     }
     wave_lds_order();
-    float total = 0.f;
+    if (ch != sc) {
+        for (int e = lane; e < E; e += 64) ch[e] = sc[e] + (a.correction ? a.correction[e] : 0.f);
+        wave_lds_order();
+    }
+    if (a.groups > 1) {
+        const int size = E / a.groups;
+        for (int g = lane; g < a.groups; g += 64) {
+            float m = -INFINITY;
+            for (int i = 0; i < size; ++i) m = fmaxf(m, ch[g * size + i]);
+            gb[g] = m;
+        }
+        wave_lds_order();
+        // a group is eligible if fewer than `keep` groups come before it (a larger best, or as large and a lower index)
+        for (int g = lane; g < a.groups; g += 64) {
+            int before = 0;
+            for (int o = 0; o < a.groups; ++o) before += gb[o] > gb[g] || (gb[o] == gb[g] && o < g);
+            if (before >= a.keep)
+                for (int i = 0; i < size; ++i) ch[g * size + i] = -INFINITY;
+        }
+        wave_lds_order();
+    }
+    float total = 0.f, id_total = 0.f;
     for (int k = 0; k < top; ++k) {
         float best = -INFINITY;
         int at = 0x7fffffff;
         for (int e = lane; e < E; e += 64) {
-            const float v = sc[e];
+            const float v = ch[e];
             if (v > best) { best = v; at = e; }
         }
 #pragma unroll
@@ -79,26 +118,40 @@ __global__ __launch_bounds__(256) void moe_route_kernel(const TI* __restrict__ x
             if (ob > best || (ob == best && oa < at)) { best = ob; at = oa; }
         }
         if (at == 0x7fffffff) at = k < E ? k : 0;     // scores that are no numbers: some expert all the same
-        total += best;
+        const float s = sc[at];
+        total += s;
+        const bool expert = at < E - a.identity;
+        if (!expert) id_total += s;
+        wave_lds_order();
         if (lane == 0) {
-            ids[(size_t)t * top + k] = at;
-            wts[(size_t)t * top + k] = best;
-            sc[at] = -INFINITY;
+            a.ids[(size_t)t * top + k] = expert ? at : -1;
+            a.wts[(size_t)t * top + k] = s;
+            ch[at] = -INFINITY;
         }
         wave_lds_order();
     }
-    if (renorm && lane == 0)
-        for (int k = 0; k < top; ++k) wts[(size_t)t * top + k] /= total;
+    const float f = (a.renorm ? 1.0f / (total + a.renorm_eps) : 1.0f) * a.out_scale;
+    if (lane == 0) {
+        if (a.renorm || a.out_scale != 1.0f)
+            for (int k = 0; k < top; ++k) a.wts[(size_t)t * top + k] *= f;
+        if (a.id_wts) a.id_wts[t] = id_total * f;
+    }
 }
 
 extern "C" int vt_moe_route(const void* x, int dtype, const float* wr, int* ids, float* wts, int n, int E, int W, int top,
-                            int softmax, int renorm, hipStream_t stream) {
+                            int softmax, int renorm, float renorm_eps, float out_scale, const float* correction, int groups,
+                            int keep, int identity, float* id_wts, hipStream_t stream) {
     VT_REQUIRE(n >= 0 && E > 0 && W > 0 && top > 0 && top <= E, "vt_moe_route: bad sizes n=%d E=%d W=%d top=%d", n, E, W, top);
-    VT_REQUIRE(E + W <= 16000, "vt_moe_route: %d experts and a width of %d (together up to 16000)", E, W);
+    VT_REQUIRE(groups >= 1 && E % groups == 0 && keep >= 1 && keep <= groups && top <= keep * (E / groups),
+               "vt_moe_route: %d of %d groups of %d experts, %d chosen", keep, groups, E, top);
+    VT_REQUIRE(identity >= 0 && identity < E && (identity == 0 || id_wts), "vt_moe_route: %d of %d outputs without an expert", identity, E);
+    const size_t floats = (size_t)W + E + (correction || groups > 1 ? E + groups : 0);
+    VT_REQUIRE(floats <= 16000, "vt_moe_route: %d experts and a width of %d (the scores and the token together up to 16000 floats)", E, W);
     if (n == 0) return 0;
-    const size_t lds = (size_t)(E + W) * sizeof(float);
-    if (dtype == VT_F32) moe_route_kernel<float><<<n, 256, lds, stream>>>((const float*)x, wr, ids, wts, E, W, top, softmax, renorm);
-    else if (dtype == VT_BF16) moe_route_kernel<bf16_t><<<n, 256, lds, stream>>>((const bf16_t*)x, wr, ids, wts, E, W, top, softmax, renorm);
+    RouteArgs a = {x, wr, correction, ids, wts, id_wts, E, W, top, softmax, renorm, groups, keep, identity, renorm_eps, out_scale};
+    const size_t lds = floats * sizeof(float);
+    if (dtype == VT_F32) moe_route_kernel<float><<<n, 256, lds, stream>>>(a);
+    else if (dtype == VT_BF16) moe_route_kernel<bf16_t><<<n, 256, lds, stream>>>(a);
     else return vt_fail("vt_moe_route: unknown dtype %d", dtype);
     VT_CHECK_LAUNCH("vt_moe_route");
     return 0;
@@ -140,6 +193,7 @@ __global__ __launch_bounds__(256) void moe_gate_up_kernel(const TI* __restrict__
     const int p = blockIdx.x;
     const int t = p / top;
     const int e = ids[p];
+    if (e < 0) return;
     const float s = scale_input ? wts[p] : 1.0f;
     for (int j = threadIdx.x; j < W; j += 256) {
         float v = load_f32<TI>(x, (size_t)t * W + j) * s;
@@ -176,6 +230,7 @@ __global__ __launch_bounds__(256) void moe_down_kernel(const TI* __restrict__ ac
     for (int k = 0; k < top; ++k) {
         const int p = t * top + k;
         const int e = ids[p];
+        if (e < 0) continue;            // (the same for the whole block)
         const float s = scale_output ? wts[p] : 1.0f;
         __syncthreads();
         for (int f = threadIdx.x; f < F; f += 256) as[f] = load_f32<TI>(act, (size_t)p * F + f);
@@ -272,7 +327,8 @@ __global__ __launch_bounds__(1024) void moe_sort_kernel(const int* __restrict__ 
     const int tid = threadIdx.x;
     for (int e = tid; e < E; e += 1024) cnt[e] = 0;
     __syncthreads();
-    for (int p = tid; p < P; p += 1024) atomicAdd(&cnt[ids[p]], 1);
+    for (int p = tid; p < P; p += 1024)
+        if (ids[p] >= 0) atomicAdd(&cnt[ids[p]], 1);
     __syncthreads();
     const int c = tid < E ? cnt[tid] : 0;
     const int tiles = (c + GR_TB - 1) / GR_TB;
@@ -298,10 +354,11 @@ __global__ __launch_bounds__(1024) void moe_sort_kernel(const int* __restrict__ 
     }
     if (tid == 1023) plan[0] = (int)(incl >> 32);
     __syncthreads();
-    for (int p = tid; p < P; p += 1024) order[atomicAdd(&cur[ids[p]], 1)] = p;
+    for (int p = tid; p < P; p += 1024)
+        if (ids[p] >= 0) order[atomicAdd(&cur[ids[p]], 1)] = p;
 }
 
-// ids [pairs] with values in [0, E); plan: vt_moe_plan_size(pairs, E) ints
+// ids [pairs] with values below E (a negative one is no pair: it is left out of the order); plan: vt_moe_plan_size(pairs, E) ints
 extern "C" int vt_moe_sort(const int* ids, int* plan, int pairs, int E, hipStream_t stream) {
     VT_REQUIRE(pairs >= 0 && E > 0 && E <= GR_MAX_EXPERTS, "vt_moe_sort: %d pairs, %d experts (up to %d)", pairs, E, GR_MAX_EXPERTS);
     if (pairs == 0) return 0;
@@ -619,23 +676,24 @@ extern "C" int vt_moe_gate_up_grouped(const void* x, const void* w_gu, const int
 }
 
 // out [n][W] float32 <- the sum over a token's choices of W_down,e act; act (sorted order) [n * top][F], w_down [E][W][F];
-// y: float32 scratch [n * top][W], needed when top > 1
+// y: float32 scratch [n * top][W], needed when top > 1 or out is null.  out null: the choices' results stay in y, in the
+// pairs' order and not added up (whoever adds them leaves out the pairs without an expert, whose rows are not written).
 extern "C" int vt_moe_down_grouped(const void* act, const void* w_down, const int* plan, const float* wts, float* out, float* y,
                                    int n, int E, int W, int F, int top, int scale_output, hipStream_t stream) {
     VT_REQUIRE(n >= 0 && E > 0 && E <= GR_MAX_EXPERTS && top > 0, "vt_moe_down_grouped: bad sizes");
     VT_REQUIRE(W > 0 && F > 0 && W % 8 == 0 && F % 8 == 0, "vt_moe_down_grouped: width %d and experts' size %d (multiples of 8)", W, F);
     VT_REQUIRE(!(((uintptr_t)act | (uintptr_t)w_down | (uintptr_t)out | (uintptr_t)y) & 15), "vt_moe_down_grouped: operands must be 16-byte aligned");
-    VT_REQUIRE(top == 1 || y, "vt_moe_down_grouped: %d choices per token need scratch", top);
+    VT_REQUIRE((top == 1 && out) || y, "vt_moe_down_grouped: %d choices per token need scratch", top);
     if (n == 0) return 0;
     if (grouped_ready()) return -1;
     const int P = n * top, T = vt_moe_plan_tiles(P, E);
     VT_REQUIRE(T <= 65535, "vt_moe_down_grouped: too many pairs (%d)", P);
-    GroupedArgs a = {(const bf16_t*)act, (const bf16_t*)w_down, plan, wts, top == 1 ? (void*)out : (void*)y, P, F, W, top, T,
+    GroupedArgs a = {(const bf16_t*)act, (const bf16_t*)w_down, plan, wts, top == 1 && out ? (void*)out : (void*)y, P, F, W, top, T,
                      scale_output, 1.f, 0.f};
     if (P <= GR_FEW_PAIRS) moe_few_kernel<false><<<dim3((W + 15) / 16, T), 256, 0, stream>>>(a);
     else moe_grouped_kernel<false><<<dim3((W + GR_FB - 1) / GR_FB, T), 256, GR_LDS_BYTES, stream>>>(a);
     VT_CHECK_LAUNCH("vt_moe_down_grouped");
-    if (top > 1) {
+    if (top > 1 && out) {
         const long long total4 = (long long)n * (W / 4);
         long long blocks = (total4 + 255) / 256;
         if (blocks > 16384) blocks = 16384;

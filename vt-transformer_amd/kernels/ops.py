@@ -867,6 +867,40 @@ def qk_prepare(x: torch.Tensor, cos: Optional[torch.Tensor], sin: Optional[torch
          _ptr(v_lambda if vmix == 2 else None), _ptr(q_gain), _ptr(k_gain), _stream())
 
 
+def qk_prepare_whole(x: torch.Tensor, positions: torch.Tensor, tok_entry: torch.Tensor, block_table: Optional[torch.Tensor],
+                     q_out: torch.Tensor, k_pages: Optional[torch.Tensor], v_pages: Optional[torch.Tensor], n_heads: int,
+                     n_kv: int, key_dim: int, value_dim: int, eps: float, q_gain: torch.Tensor,
+                     k_gain: Optional[torch.Tensor], write_kv: bool = True) -> None:
+    """qk_prepare for queries and keys that are normed over the whole projection: the H D query elements of a token are
+    divided by their common root mean square (eps inside the root) and multiplied by q_gain (float32 [H * D]), the G D
+    key elements by theirs and k_gain.  x [n, >= H D] or, with write_kv, [n, >= (H + G) D + G Dv]; the layouts are
+    qk_prepare's."""
+    n = x.shape[0]
+    _chk(x, "qk_prepare_whole.x")
+    need = (n_heads + (n_kv if write_kv else 0)) * key_dim + (n_kv * value_dim if write_kv else 0)
+    if x.dim() != 2 or x.shape[1] < need:
+        raise KernelError(f"qk_prepare_whole.x: shape {tuple(x.shape)}, need {need} columns")
+    _chk(positions, "qk_prepare_whole.positions", torch.int32, (n,))
+    _chk(tok_entry, "qk_prepare_whole.tok_entry", torch.int32, (n,))
+    _chk(q_out, "qk_prepare_whole.q_out", None, (n, n_heads * key_dim))
+    _chk(q_gain, "qk_prepare_whole.q_gain", torch.float32, (n_heads * key_dim,))
+    if x.dtype != torch.float32 and x.dtype != q_out.dtype:
+        raise KernelError(f"qk_prepare_whole: {x.dtype} inputs and {q_out.dtype} queries")
+    page_size = num_pages = max_blocks = 0
+    if write_kv:
+        _chk(k_gain, "qk_prepare_whole.k_gain", torch.float32, (n_kv * key_dim,))
+        num_pages, page_size = k_pages.shape[0], k_pages.shape[2]
+        _chk(k_pages, "qk_prepare_whole.k_pages", q_out.dtype, (num_pages, n_kv, page_size, key_dim))
+        _chk(v_pages, "qk_prepare_whole.v_pages", q_out.dtype, (num_pages, n_kv, value_dim, page_size))
+        _chk(block_table, "qk_prepare_whole.block_table", torch.int32)
+        max_blocks = block_table.shape[1]
+    _run(load_lib("vt_attn_masked", half=_half(x, q_out)), "vt_qk_prepare_whole", _ptr(x), _i(_code(x)),
+         ctypes.c_longlong(x.stride(0)), _ptr(positions), _ptr(tok_entry), _ptr(block_table if write_kv else None),
+         _i(max_blocks), _ptr(q_out), _ptr(k_pages if write_kv else None), _ptr(v_pages if write_kv else None),
+         _i(_code(q_out)), _i(page_size), _i(num_pages), _i(n), _i(n_heads), _i(n_kv), _i(key_dim), _i(value_dim),
+         _i(1 if write_kv else 0), _f(eps), _ptr(q_gain), _ptr(k_gain if write_kv else None), _stream())
+
+
 def attention_masked(q: torch.Tensor, k_pages: torch.Tensor, v_pages: torch.Tensor, positions: torch.Tensor,
                      tok_entry: torch.Tensor, block_table: torch.Tensor, out: torch.Tensor, n_heads: int, n_kv: int,
                      key_dim: int, value_dim: int, scale: float, cap: float = 0.0, window: int = 0, chunk: int = 0,
@@ -1440,10 +1474,17 @@ def token_shift(h: torch.Tensor, mu: torch.Tensor, state: torch.Tensor, tok_entr
 # ---------------------------------------------------------------------------
 # a feed-forward of many experts (vt_moe.hip)
 def moe_route(x: torch.Tensor, router: torch.Tensor, ids: torch.Tensor, weights: torch.Tensor, score: str = "sigmoid",
-              renormalize: bool = False) -> None:
+              renormalize: bool = False, renorm_eps: float = 0.0, out_scale: float = 1.0,
+              correction: Optional[torch.Tensor] = None, groups: int = 1, keep: int = 1, identity: int = 0,
+              identity_weights: Optional[torch.Tensor] = None) -> None:
     """ids[t], weights[t] <- the `top` experts with the largest scores of token t and those scores (the largest
     first, the lower index among equals); scores are sigmoid or softmax of router x, in float32; renormalize: the
-    chosen scores are divided by their sum.  x [n, W], router [E, W] float32, ids [n, top] int32, weights [n, top]."""
+    chosen scores are divided by their sum + renorm_eps; out_scale: and then multiplied by this.  x [n, W], router
+    [E, W] float32, ids [n, top] int32, weights [n, top].
+    correction (float32 [E]): added to the scores for the choice, not to the weights.  groups, keep: the E outputs are
+    `groups` runs of neighbours, and only those of the `keep` groups with the largest choice score in them can be
+    chosen.  identity: the last so many outputs are no experts: a chosen one has the id -1, and its weight is added to
+    identity_weights[t] (float32 [n], zero where none is chosen)."""
     n, w = x.shape
     e = router.shape[0]
     _chk(x, "moe_route.x")
@@ -1453,14 +1494,19 @@ def moe_route(x: torch.Tensor, router: torch.Tensor, ids: torch.Tensor, weights:
     _chk(weights, "moe_route.weights", torch.float32, (n, top))
     if score not in ("sigmoid", "softmax") or not 1 <= top <= e:
         raise KernelError(f"moe_route: score {score!r}, {top} of {e} experts")
+    if correction is not None:
+        _chk(correction, "moe_route.correction", torch.float32, (e,))
+    if identity_weights is not None:
+        _chk(identity_weights, "moe_route.identity_weights", torch.float32, (n,))
     _run(load_lib("vt_moe", half=_half(x)), "vt_moe_route", _ptr(x), _i(_code(x)), _ptr(router), _ptr(ids), _ptr(weights),
-         _i(n), _i(e), _i(w), _i(top), _i(1 if score == "softmax" else 0), _i(1 if renormalize else 0), _stream())
+         _i(n), _i(e), _i(w), _i(top), _i(1 if score == "softmax" else 0), _i(1 if renormalize else 0), _f(renorm_eps),
+         _f(out_scale), _ptr(correction), _i(groups), _i(keep), _i(identity), _ptr(identity_weights), _stream())
 
 
 def moe_gate_up(x: torch.Tensor, w_gu: torch.Tensor, ids: torch.Tensor, weights: torch.Tensor, act: torch.Tensor,
                 scale_input: bool, alpha: float = 1.0, cubic: float = 0.0) -> torch.Tensor:
     """act[t * top + k] = f(W_gate,e xe) * (W_up,e xe) for e = ids[t, k], xe = x[t] (times weights[t, k] if
-    scale_input, rounded to x's type), f(g) = g sigmoid(alpha g (1 + cubic g^2)); w_gu [E, 2 F, W] (gate rows, then up
+    scale_input, rounded to x's type; a pair whose id is negative is left out), f(g) = g sigmoid(alpha g (1 + cubic g^2)); w_gu [E, 2 F, W] (gate rows, then up
     rows); act [n * top, F] in x's type.  An expert's matrices are read once per token that chose it."""
     n, w = x.shape
     e, two_f, _ = w_gu.shape
@@ -1478,7 +1524,8 @@ def moe_gate_up(x: torch.Tensor, w_gu: torch.Tensor, ids: torch.Tensor, weights:
 
 def moe_down(act: torch.Tensor, w_down: torch.Tensor, ids: torch.Tensor, weights: torch.Tensor, out: torch.Tensor,
              scale_output: bool) -> torch.Tensor:
-    """out[t] = sum_k (weights[t, k] if scale_output) * W_down,e act[t * top + k], e = ids[t, k], in the order of k;
+    """out[t] = sum_k (weights[t, k] if scale_output) * W_down,e act[t * top + k], e = ids[t, k], in the order of k
+    (without the pairs whose id is negative);
     w_down [E, W, F]; out [n, W] float32."""
     e, w, f = w_down.shape
     n, top = ids.shape
@@ -1509,7 +1556,7 @@ def moe_grouped_ok(x: torch.Tensor, experts: int, width: int, inter: int) -> boo
 
 def moe_sort(ids: torch.Tensor, plan: torch.Tensor, experts: int) -> torch.Tensor:
     """plan <- the pairs in the order of their experts, cut into tiles of pairs of one expert (what the grouped
-    products read).  ids [n, top] int32 with values below `experts`; plan: moe_plan_size(n * top, experts) int32."""
+    products read).  ids [n, top] int32 with values below `experts` (a negative one is left out); plan: moe_plan_size(n * top, experts) int32."""
     _chk(ids, "moe_sort.ids", torch.int32)
     pairs = ids.numel()
     _chk(plan, "moe_sort.plan", torch.int32, (moe_plan_size(pairs, experts),))
@@ -1535,10 +1582,11 @@ def moe_gate_up_grouped(x: torch.Tensor, w_gu: torch.Tensor, plan: torch.Tensor,
     return act
 
 
-def moe_down_grouped(act: torch.Tensor, w_down: torch.Tensor, plan: torch.Tensor, weights: torch.Tensor, out: torch.Tensor,
-                     scratch: Optional[torch.Tensor], scale_output: bool) -> torch.Tensor:
+def moe_down_grouped(act: torch.Tensor, w_down: torch.Tensor, plan: torch.Tensor, weights: torch.Tensor,
+                     out: Optional[torch.Tensor], scratch: Optional[torch.Tensor], scale_output: bool) -> torch.Tensor:
     """moe_down on the matrix cores from activations in the plan's order; scratch [n * top, W] float32 where a token
-    has more than one choice (the choices' results, added in their order afterwards)."""
+    has more than one choice (the choices' results, added in their order afterwards).  out None: the choices' results
+    are left in `scratch`, a row per (token, choice), not added up (`sublayer_sum` and `output_norm_add` do that)."""
     e, w, f = w_down.shape
     n, top = weights.shape
     _chk(act, "moe_down_grouped.act", None, (n * top, f))
@@ -1547,14 +1595,71 @@ def moe_down_grouped(act: torch.Tensor, w_down: torch.Tensor, plan: torch.Tensor
     _chk(w_down, "moe_down_grouped.w_down", act.dtype)
     _chk(plan, "moe_down_grouped.plan", torch.int32, (moe_plan_size(n * top, e),))
     _chk(weights, "moe_down_grouped.weights", torch.float32)
-    _chk(out, "moe_down_grouped.out", torch.float32, (n, w))
-    if top > 1:
+    needs_scratch = top > 1 or out is None
+    if out is not None:
+        _chk(out, "moe_down_grouped.out", torch.float32, (n, w))
+    if needs_scratch:
         if scratch is None:
             raise KernelError("moe_down_grouped: several choices per token need scratch")
         _chk(scratch, "moe_down_grouped.scratch", torch.float32, (n * top, w))
     _run(load_lib("vt_moe", half=_half(act)), "vt_moe_down_grouped", _ptr(act), _ptr(w_down), _ptr(plan), _ptr(weights), _ptr(out),
-         _ptr(scratch if top > 1 else None), _i(n), _i(e), _i(w), _i(f), _i(top), _i(1 if scale_output else 0), _stream())
+         _ptr(scratch if needs_scratch else None), _i(n), _i(e), _i(w), _i(f), _i(top), _i(1 if scale_output else 0), _stream())
+    return out if out is not None else scratch
+
+
+# ---------------------------------------------------------------------------
+# a sublayer's result, whole or in pieces, and the norm on it (vt_output_norm.hip)
+def _pieces(who: str, n: int, w: int, y, choices, ids, id_weights, x):
+    """Checks of the pieces of a sublayer's result; returns the arguments that describe them."""
+    top = 0
+    if choices is not None:
+        _chk(choices, who + ".choices", torch.float32)
+        if choices.dim() != 2 or choices.shape[1] != w or n == 0 or choices.shape[0] % n:
+            raise KernelError(f"{who}.choices: shape {tuple(choices.shape)} is not a row of {w} per choice of {n} tokens")
+        top = choices.shape[0] // n
+        if ids is not None:
+            _chk(ids, who + ".ids", torch.int32, (n, top))
+    if id_weights is not None:
+        _chk(id_weights, who + ".id_weights", torch.float32, (n,))
+        _chk(x, who + ".x", None, (n, w))
+    if y is not None:
+        _chk(y, who + ".y", None, (n, w))
+    if choices is None and id_weights is None and y is None:
+        raise KernelError(who + ": no pieces")
+    return (_ptr(choices), _ptr(ids if choices is not None else None), _i(top), _ptr(id_weights),
+            _ptr(x if id_weights is not None else None), _i(_code(x) if id_weights is not None else F32), _ptr(y),
+            _i(_code(y) if y is not None else F32))
+
+
+def sublayer_sum(out: torch.Tensor, y: Optional[torch.Tensor] = None, choices: Optional[torch.Tensor] = None,
+                 ids: Optional[torch.Tensor] = None, id_weights: Optional[torch.Tensor] = None,
+                 x: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """out[t] = sum_k choices[t * top + k] + id_weights[t] * x[t] + y[t], every kind of piece optional: choices float32
+    [n * top, W], of which those with a negative id (ids int32 [n, top]; None: all count) are left out; x and y [n, W]
+    float32 or 16-bit; out [n, W] float32."""
+    n, w = out.shape
+    _chk(out, "sublayer_sum.out", torch.float32)
+    args = _pieces("sublayer_sum", n, w, y, choices, ids, id_weights, x)
+    _run(load_lib("vt_output_norm", half=_half(x if id_weights is not None else None, y)), "vt_sublayer_sum", _ptr(out), *args, _i(n),
+         _i(w), _stream())
     return out
+
+
+def output_norm_add(h: torch.Tensor, gain: torch.Tensor, eps: float, mult: float, y: Optional[torch.Tensor] = None,
+                    choices: Optional[torch.Tensor] = None, ids: Optional[torch.Tensor] = None,
+                    id_weights: Optional[torch.Tensor] = None, x: Optional[torch.Tensor] = None,
+                    copy: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """h[t] += mult * gain * u[t] / sqrt(mean(u[t]^2) + eps) with u what `sublayer_sum` gives for the same pieces (x may
+    be h itself); h float32 [n, W], changed in place.  copy [n, W]: the new h in this tensor's type as well."""
+    n, w = h.shape
+    _chk(h, "output_norm_add.h", torch.float32)
+    _chk(gain, "output_norm_add.gain", torch.float32, (w,))
+    if copy is not None:
+        _chk(copy, "output_norm_add.copy", None, (n, w))
+    args = _pieces("output_norm_add", n, w, y, choices, ids, id_weights, x)
+    _run(load_lib("vt_output_norm", half=_half(x if id_weights is not None else None, y, copy)), "vt_output_norm_add", _ptr(h), *args,
+         _ptr(gain), _ptr(copy), _i(_code(copy) if copy is not None else F32), _i(n), _i(w), _f(mult), _f(eps), _stream())
+    return h
 
 
 # ---------------------------------------------------------------------------

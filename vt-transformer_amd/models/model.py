@@ -16,7 +16,7 @@ from ..config.base import LayerSpec, ModelSpec, PartSpec
 from ..kernels import ops
 from ..parts.linear import linear
 from ..parts.base import (BLOCKS, EMBEDDINGS, FEED_FORWARDS, HEADS, MIXERS, NORMS, NormedInput, Part, Registry,
-                          Runtime, TensorDecl)
+                          Runtime, StreamCopy, TensorDecl)
 
 
 def settle(h: torch.Tensor, delta):
@@ -122,6 +122,8 @@ class DecoderModel:
         last = len(self.schedule) - 1
         for i, entry in enumerate(self.schedule):
             block = self.layers[entry.layer]
+            if isinstance(delta, StreamCopy) and not getattr(block, "takes_stream_copy", False):
+                delta = None                # (nothing is left to be added; this block goes on from the stream)
             if isinstance(delta, tuple) and (entry.inject or entry.offset_row is not None
                                              or not getattr(block, "takes_pair", False)):
                 h, delta = settle(h, delta), None
@@ -150,7 +152,7 @@ class DecoderModel:
                 h, delta = block.forward(h, delta, ctx, caches[i], states[i])
         if ctx.n_logit_rows == 0:
             return None
-        if isinstance(delta, NormedInput):
+        if isinstance(delta, (NormedInput, StreamCopy)):
             delta = None
         if isinstance(delta, tuple):
             if getattr(self.final_norm, "takes_pair", False) and not self.streams:

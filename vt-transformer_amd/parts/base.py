@@ -10,6 +10,8 @@ Interfaces (N = tokens of the step, H = model width):
 
   Norm            forward(h[N,H] fp32, delta[N,H] or None, rows=None) -> normed [N or R, H] in the runtime's dtype.
                   With `delta`, h += delta happens first (and is stored in h unless `rows` picks rows).
+                  Optional: forward_output(h, y, mult, copy), the norm on a sublayer's output: h += mult * norm(y), with
+                  y a tensor or SublayerPieces, and the new h in `copy` as well.
   PositionEncoding
                   rotary_tables(n_positions) -> (cos, sin) fp32 [n_positions, dims/2] or None if the
                   encoding is not a rotation that the fused kernel can apply;
@@ -19,14 +21,16 @@ Interfaces (N = tokens of the step, H = model width):
                   Optional: prepare_step(ctx) -> {key: int32 array} or None, called on the host once per step
                   before the step's metadata goes to the device; what it returns is found in ctx.extra[key] on
                   the device when the part runs (work items of its kernels, lengths they read from memory).
-  FeedForward     forward(x[N,H], ctx) -> [N,H]
+  FeedForward     forward(x[N,H], ctx) -> [N,H].  One that `hands_pieces` takes pieces=True and may then return its
+                  result not added up (SublayerPieces).
   Embedding       forward(ids[N] int32) -> h[N,H] fp32; `name` and `table` say what it has loaded.
   Head            load(get, rt, shared) where `shared` maps tensor names to tensors that other parts have placed
                   on the device already (a tied head finds the embedding's table there); forward(x[R,H]) -> fp32
                   logits [R,V].
   Block           forward(h, delta, ctx, cache, state) -> (h, delta): arranges two norms, a mixer and a
                   feed-forward around the fp32 residual stream h.  `delta` is a layer output that has
-                  not been added to h yet, so that the next norm can fuse the addition.
+                  not been added to h yet, so that the next norm can fuse the addition (or None, or what a
+                  block of its kind can use: NormedInput, a pair of tensors, StreamCopy).
 
 The reference's counterpart is the set of `op.*` words that a model program
 strings together (v1/tensortype/nn_operators.cpp:530-576) and its user words
@@ -220,6 +224,35 @@ class NormedInput:
 
     def materialize(self) -> torch.Tensor:
         return self.norm.forward(self.h, None)
+
+
+class StreamCopy:
+    """What a block whose sublayers read the residual stream itself hands on instead of an addend: nothing is left to be
+    added to the stream, and `x` is the stream in the runtime's dtype (the stream itself in float32), as the norm on its
+    last sublayer's output has written it.  Whoever does not read it goes on from the stream."""
+
+    def __init__(self, x: torch.Tensor):
+        self.x = x
+
+
+class SublayerPieces:
+    """A sublayer's result that has not been added up: rows of a mixture's choices [tokens * top, width] (those with a
+    negative id left out), a weight per token on the sublayer's own input, and a result that every token has, each
+    optional.  A norm on the output takes the pieces as they are (`RMSNorm.forward_output`); `materialize()` is their
+    sum as a tensor, for whoever cannot."""
+
+    def __init__(self, rt: "Runtime", rows: int, width: int, y: Optional[torch.Tensor] = None,
+                 choices: Optional[torch.Tensor] = None, ids: Optional[torch.Tensor] = None,
+                 id_weights: Optional[torch.Tensor] = None, x: Optional[torch.Tensor] = None):
+        self.rt, self.rows, self.width = rt, int(rows), int(width)
+        self.y, self.choices, self.ids, self.id_weights, self.x = y, choices, ids, id_weights, x
+
+    def as_args(self) -> Dict[str, Optional[torch.Tensor]]:
+        return dict(y=self.y, choices=self.choices, ids=self.ids, id_weights=self.id_weights, x=self.x)
+
+    def materialize(self) -> torch.Tensor:
+        from ..kernels import ops
+        return ops.sublayer_sum(self.rt.buffer("pieces.sum", (self.rows, self.width), torch.float32), **self.as_args())
 
 
 class HostStaging:

@@ -22,7 +22,7 @@ from typing import Callable, Dict, Optional, Tuple
 import torch
 
 from ..kernels import ops
-from .base import BLOCKS, NormedInput, Part, Runtime, StateNeed, TensorDecl
+from .base import BLOCKS, NormedInput, Part, Runtime, StateNeed, StreamCopy, TensorDecl
 from .linear import can_fuse, linear
 
 
@@ -130,6 +130,57 @@ class ParallelBlock(Part):
             ops.residual_add(h, y)
             return h, z
         return h, (y, z)
+
+
+@BLOCKS.register("output_norm")
+class OutputNormBlock(Part):
+    """No norm in front of the sublayers: they read the residual stream x itself, and what is normed is their result,
+
+        x <- x + m * norm_1(mixer(x));   x <- x + m * norm_2(feed_forward(x))
+
+    with m a constant (`residual_mult`).  Norm, factor, addition and the copy of the stream in the runtime's dtype that
+    the next sublayer's products read are one kernel (`forward_output`), which also adds up the pieces of a feed-forward
+    that hands them on so.  The block passes the copy on to the block behind it (StreamCopy)."""
+
+    norm_roles = ("mixer_output", "feed_forward_output")
+    replayable = True
+    takes_stream_copy = True    # forward(h, delta, ...) with delta a StreamCopy: h in the runtime's dtype is there already
+
+    def __init__(self, *, rt: Runtime, norms, mixer, feed_forward, prefix: str = "", width: int = 0, residual_mult: float = 1.0,
+                 idle_norm: Optional[str] = None):
+        """residual_mult: the factor m; idle_norm: the second norm's tensor of a layer without a feed-forward, which a
+        checkpoint may hold and which is not read."""
+        self.rt, self.width = rt, int(width)
+        self.mult = float(residual_mult)
+        self.idle_norm = prefix + idle_norm if idle_norm is not None and feed_forward is None else None
+        self.norm_mixer = norms["mixer_output"]
+        self.mixer = mixer
+        self.feed_forward = feed_forward
+        self.norm_ff = norms["feed_forward_output"] if feed_forward is not None else None
+
+    def parts(self):
+        if self.feed_forward is None:
+            return [self, self.mixer, self.norm_mixer]
+        return [self, self.mixer, self.norm_mixer, self.feed_forward, self.norm_ff]
+
+    def tensors(self) -> Dict[str, TensorDecl]:
+        return {self.idle_norm: TensorDecl((self.width,), "bias", optional=True)} if self.idle_norm is not None else {}
+
+    def forward(self, h: torch.Tensor, delta, ctx, cache, state) -> Tuple[torch.Tensor, object]:
+        rt = self.rt
+        copy = rt.buffer("stream.copy", tuple(h.shape), rt.dtype) if rt.lowp else None
+        if isinstance(delta, StreamCopy):
+            x = delta.x
+        else:
+            if isinstance(delta, torch.Tensor):
+                ops.residual_add(h, delta)
+            x = ops.gather_rows(h, None, copy) if rt.lowp else h
+        self.norm_mixer.forward_output(h, self.mixer.forward(x, ctx, cache, state), self.mult, copy)
+        x = copy if rt.lowp else h
+        if self.feed_forward is not None:
+            more = {"pieces": True} if getattr(self.feed_forward, "hands_pieces", False) else {}
+            self.norm_ff.forward_output(h, self.feed_forward.forward(x, ctx, **more), self.mult, copy)
+        return h, StreamCopy(x)
 
 
 @BLOCKS.register("hyper")

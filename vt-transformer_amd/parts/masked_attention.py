@@ -8,8 +8,9 @@ one sigmoid gate per head (or per element) on the output, a gain on the
 unit-RMS queries and keys, a bias that grows with the logarithm of the
 distance, a learned shift of every score per head, weights that are sigmoids of
 the scores instead of a softmax, neighbouring elements rotated together, a bias
-on the output projection.  Every one of these is a constructor parameter that
-can be left out.
+on the output projection, queries and keys normed over the whole projection
+before it is split into heads, keys and values taken from an earlier layer's
+pages.  Every one of these is a constructor parameter that can be left out.
 
 Per token: q, k, v (and the gates' logits) in one matrix product with the
 biases; rotation, unit scaling and the write into the pages in one kernel;
@@ -27,11 +28,15 @@ reads the pages; output projection.
     score_shift:   score(i, j) += shift_h                              learned, one per head
     weights "sigmoid":  p_ij = sigmoid(score(i, j)) for every seen j, not normalized (no sink)
     out_gate:      out_i[h][d] *= sigmoid((W_g x_i)[h][d])             one logit per output element instead of per head
+    whole norm:    q <- gain * q / sqrt(mean(q^2) + eps) over all rows of W_q x at once (and k likewise over W_k x)
     qk_gain:       after the unit-RMS scaling q and k are multiplied by a learned gain per element (shared by heads)
 
 Value mixing ties layers together: the first layer of a model that says value_mix="source" leaves the step's values
 in a buffer, and every layer that says value_mix="mix" keeps (1 - lambda) v + lambda v_source in its pages instead
 of its own v, with lambda a learned number of its own.
+
+A layer that takes another layer's keys and values (its schedule entry names that layer's cache) has queries, mask
+and scores of its own and writes nothing: its pages are the other layer's, as that layer left them.
 
 Chunks are counted from position 0 of the sequence.  A key that no later
 position can see is dead for the cache manager: the pages' window is the
@@ -110,7 +115,8 @@ class MaskedAttention(Part):
                  names: Optional[Dict[str, str]] = None, sink: bool = False, distance_slopes: Optional[float] = None,
                  q_temp: Optional[Dict[str, float]] = None, value_mix: Optional[str] = None, fuse_norms: bool = False,
                  rot_pairs: str = "halves", qk_gain: bool = False, distance_log: bool = False, score_shift: bool = False,
-                 weights: str = "softmax", out_gate: bool = False, o_bias: bool = False):
+                 weights: str = "softmax", out_gate: bool = False, o_bias: bool = False,
+                 whole_norm_eps: Optional[float] = None, own_keys: bool = True):
         """key_dim / value_dim: sizes of a head's queries and keys / of its values (default: the same);
         position: a rotary encoding whose `dim` may be smaller than key_dim (the rest of a head passes unchanged);
         unit_rms_eps: queries and keys are divided by their root mean square per head after the rotation, with
@@ -130,14 +136,19 @@ class MaskedAttention(Part):
         rotation is the neighbouring one, and a score, a sum over the elements of q and k alike, does not see the
         order); qk_gain (with unit_rms_eps): tensors q_norm, k_norm [key_dim]; distance_log: tensors r1, r2 [heads];
         score_shift: tensor shift [heads]; weights: "softmax" or "sigmoid"; out_gate: an elementwise sigmoid gate from
-        a projection g [heads * value_dim, width] (head_gate's tensor name; not both); o_bias: tensor o_bias [width]."""
+        a projection g [heads * value_dim, width] (head_gate's tensor name; not both); o_bias: tensor o_bias [width];
+            whole_norm_eps: queries and keys are divided by the root mean square of the whole projection (eps inside the
+            root), tensors q_norm [heads * key_dim] and k_norm [kv heads * key_dim] (None: they are not; without
+            rotation, query factor, value mixing and the per-head norm); own_keys False: the layer has no key and value
+            projections (and no k_norm) and reads the cache that its schedule entry names."""
         if num_heads % num_kv_heads:
             raise ValueError(f"{num_heads} query heads are not a multiple of {num_kv_heads} key/value heads")
         self.rt, self.width = rt, int(width)
         self.nh, self.nkv, self.d = int(num_heads), int(num_kv_heads), int(key_dim)
         self.dv = int(value_dim) if value_dim is not None else self.d
-        if not 1 <= self.d <= ops.MASKED_MAX_KEY_DIM or not 1 <= self.dv <= ops.MASKED_MAX_VALUE_DIM:
-            raise ValueError(f"head sizes {self.d}/{self.dv}: the kernels take keys up to {ops.MASKED_MAX_KEY_DIM} and "
+        max_d = ops.MASKED_MAX_KEY_DIM if whole_norm_eps is None else ops.ATTN_MASKED_MAX_KEY_DIM
+        if not 1 <= self.d <= max_d or not 1 <= self.dv <= ops.MASKED_MAX_VALUE_DIM:
+            raise ValueError(f"head sizes {self.d}/{self.dv}: the kernels take keys up to {max_d} and "
                              f"values up to {ops.MASKED_MAX_VALUE_DIM}")
         self.qkv_bias, self.head_gate = bool(qkv_bias), bool(head_gate)
         self.scale = float(scale) if scale is not None else 1.0 / math.sqrt(self.d)
@@ -172,6 +183,14 @@ class MaskedAttention(Part):
             raise ValueError("one gate on the output: per head or per element")
         if self.sigmoid_weights and self.has_sink:
             raise ValueError("sigmoid weights have no denominator for a sink to join")
+        self.whole_norm_eps = None if whole_norm_eps is None else float(whole_norm_eps)
+        self.own_keys = bool(own_keys)
+        if self.whole_norm_eps is not None and (self.unit_rms_eps is not None or position is not None or self.q_temp
+                                                or value_mix is not None):
+            raise ValueError("a norm over the whole projection is not combined with rotation, a query factor, value mixing "
+                             "or a norm per head")
+        if not self.own_keys and value_mix in ("source", "mix"):
+            raise ValueError("a layer that reads another layer's values has none to mix")
         # what the block asks for (parts/block.py)
         self.takes_normed_input = self.hands_norm_on = bool(fuse_norms)
         n = {"q": "q_proj.weight", "k": "k_proj.weight", "v": "v_proj.weight", "o": "o_proj.weight", "g": "g_proj.weight",
@@ -194,10 +213,10 @@ class MaskedAttention(Part):
         self.sink = self.slopes = self.v_lambda = None
         self.q_gain = self.k_gain = self.r1 = self.r2 = self.shift = self.b_o = self.b_o_lowp = None
 
-    # columns of the input projection: queries, keys, values, gates
+    # columns of the input projection: queries, keys and values (of a layer that has its own), gates
     @property
     def _gate_column(self) -> int:
-        return (self.nh + self.nkv) * self.d + self.nkv * self.dv
+        return self.nh * self.d + (self.nkv * (self.d + self.dv) if self.own_keys else 0)
 
     def cache_need(self) -> Optional[CacheNeed]:
         """Keys [kv head][slot][D] and values transposed, [kv head][Dv][slot] (the matrix-core kernel reads four keys of
@@ -224,23 +243,28 @@ class MaskedAttention(Part):
 
     def tensors(self) -> Dict[str, TensorDecl]:
         nm = self.names
-        t = {
-            nm["q"]: TensorDecl((self.nh * self.d, self.width), "matrix"),
-            nm["k"]: TensorDecl((self.nkv * self.d, self.width), "matrix"),
-            nm["v"]: TensorDecl((self.nkv * self.dv, self.width), "matrix"),
-            nm["o"]: TensorDecl((self.width, self.nh * self.dv), "matrix"),
-        }
+        t = {nm["q"]: TensorDecl((self.nh * self.d, self.width), "matrix")}
+        if self.own_keys:
+            t[nm["k"]] = TensorDecl((self.nkv * self.d, self.width), "matrix")
+            t[nm["v"]] = TensorDecl((self.nkv * self.dv, self.width), "matrix")
+        t[nm["o"]] = TensorDecl((self.width, self.nh * self.dv), "matrix")
         if self.qkv_bias:
             t[nm["q_bias"]] = TensorDecl((self.nh * self.d,), "bias")
-            t[nm["k_bias"]] = TensorDecl((self.nkv * self.d,), "bias")
-            t[nm["v_bias"]] = TensorDecl((self.nkv * self.dv,), "bias")
+            if self.own_keys:
+                t[nm["k_bias"]] = TensorDecl((self.nkv * self.d,), "bias")
+                t[nm["v_bias"]] = TensorDecl((self.nkv * self.dv,), "bias")
+        if self.whole_norm_eps is not None:
+            t[nm["q_norm"]] = TensorDecl((self.nh * self.d,), "gain")
+            if self.own_keys:
+                t[nm["k_norm"]] = TensorDecl((self.nkv * self.d,), "gain")
         if self.head_gate:
             t[nm["g"]] = TensorDecl((self.nh, self.width), "matrix")
         if self.out_gate:
             t[nm["g"]] = TensorDecl((self.nh * self.dv, self.width), "matrix")
         if self.qk_gain:
             t[nm["q_norm"]] = TensorDecl((self.d,), "gain")
-            t[nm["k_norm"]] = TensorDecl((self.d,), "gain")
+            if self.own_keys:
+                t[nm["k_norm"]] = TensorDecl((self.d,), "gain")
         if self.distance_log:
             t[nm["r1"]] = TensorDecl((self.nh,), "bias")
             # (r2 multiplies the distance inside the logarithm: a model with random weights draws it around 1)
@@ -270,18 +294,20 @@ class MaskedAttention(Part):
     def load(self, get: Callable[[str], torch.Tensor], rt: Runtime) -> None:
         nm = self.names
         gated = self.head_gate or self.out_gate
-        mats = [rt.place(get(nm[k]), "matrix") for k in (("q", "k", "v", "g") if gated else ("q", "k", "v"))]
-        mats[0], mats[1] = self._pair_order(mats[0], self.nh), self._pair_order(mats[1], self.nkv)
-        self.w_in = torch.cat(mats, dim=0).contiguous()
+        made = ["q", "k", "v"] if self.own_keys else ["q"]
+        mats = {k: rt.place(get(nm[k]), "matrix") for k in made + (["g"] if gated else [])}
+        heads = {"q": self.nh, "k": self.nkv}
+        self.w_in = torch.cat([self._pair_order(m, heads[k]) if k in heads else m for k, m in mats.items()], dim=0).contiguous()
         if self.qkv_bias:
-            b = [rt.place(get(nm[k]), "bias") for k in ("q_bias", "k_bias", "v_bias")]
-            b[0], b[1] = self._pair_order(b[0], self.nh), self._pair_order(b[1], self.nkv)
+            b = {k: rt.place(get(nm[k + "_bias"]), "bias") for k in made}
+            b = [self._pair_order(m, heads[k]) if k in heads else m for k, m in b.items()]
             if gated:
-                b.append(torch.zeros(mats[3].shape[0], dtype=torch.float32, device=rt.device))
+                b.append(torch.zeros(mats["g"].shape[0], dtype=torch.float32, device=rt.device))
             self.b_in = torch.cat(b, dim=0).contiguous()
             self.b_in_lowp = self.b_in.to(rt.dtype)
-        if self.qk_gain:
-            self.q_gain, self.k_gain = rt.place(get(nm["q_norm"]), "gain"), rt.place(get(nm["k_norm"]), "gain")
+        if self.qk_gain or self.whole_norm_eps is not None:
+            self.q_gain = rt.place(get(nm["q_norm"]), "gain")
+            self.k_gain = rt.place(get(nm["k_norm"]), "gain") if self.own_keys else None
         if self.distance_log:
             self.r1, self.r2 = rt.place(get(nm["r1"]), "bias"), rt.place(get(nm["r2"]), "gain")
         if self.score_shift:
@@ -306,17 +332,21 @@ class MaskedAttention(Part):
     def forward(self, x, ctx, cache, state=None, residual: Optional[torch.Tensor] = None, hand_on=None):
         rt, nh, nkv, d, dv = self.rt, self.nh, self.nkv, self.d, self.dv
         n = x.shape[0]
-        if not cache.writes:
-            raise RuntimeError("this mixer does not read another layer's keys and values")
+        if bool(cache.writes) != self.own_keys:
+            raise RuntimeError("a layer makes keys and values exactly if its schedule entry has a cache of its own")
         y = linear(rt, x, self.w_in, self.b_in, "mattn.in", bias_lowp=self.b_in_lowp, packed=self.p_in)
         tables = self.position.rotary_tables(ctx.n_positions) if getattr(self.position, "dim", 0) else None
         cos, sin = tables if tables is not None else (None, None)
         q = rt.buffer("mattn.q", (n, nh * d), rt.dtype)
         # the values that layers mix: one buffer per model and step, written by the source layer, read by the others
         v_first = rt.buffer("mattn.v_first", (n, nkv * dv), torch.float32) if self.value_mix in ("source", "mix") else None
-        ops.qk_prepare(y, cos, sin, ctx.positions, ctx.tok_entry, cache.block_table, q, cache["k"], cache["v"], nh, nkv,
-                       d, dv, self.unit_rms_eps, q_temp=self.q_temp, v_first=v_first, v_lambda=self.v_lambda,
-                       q_gain=self.q_gain, k_gain=self.k_gain)
+        if self.whole_norm_eps is not None:
+            ops.qk_prepare_whole(y, ctx.positions, ctx.tok_entry, cache.block_table, q, cache["k"], cache["v"], nh, nkv, d, dv,
+                                 self.whole_norm_eps, self.q_gain, self.k_gain, write_kv=self.own_keys)
+        else:
+            ops.qk_prepare(y, cos, sin, ctx.positions, ctx.tok_entry, cache.block_table, q, cache["k"], cache["v"], nh, nkv,
+                           d, dv, self.unit_rms_eps, write_kv=self.own_keys, q_temp=self.q_temp, v_first=v_first,
+                           v_lambda=self.v_lambda, q_gain=self.q_gain, k_gain=self.k_gain)
         out = rt.buffer("mattn.out", (n, nh * dv), rt.dtype)
         run_masked_attention(rt, ctx, cache, q, out, nh, nkv, d, dv, self.scale, self.softcap, self.window, self.chunk,
                              gate=y if (self.head_gate or self.out_gate) else None, gate_column=self._gate_column,

@@ -13,7 +13,7 @@ from typing import Callable, Dict, Optional
 import torch
 
 from ..kernels import ops
-from .base import NORMS, Part, Runtime, TensorDecl
+from .base import NORMS, Part, Runtime, SublayerPieces, TensorDecl
 
 
 @NORMS.register("rmsnorm")
@@ -55,6 +55,12 @@ class RMSNorm(Part):
         n = rows.numel() if rows is not None else h.shape[0]
         out = self.rt.buffer(self.scratch + (".rows" if rows is not None else ""), (n, self.width), self.rt.dtype)
         return ops.rmsnorm(h, delta, self.gain, out, self.eps, rows=rows)
+
+    def forward_output(self, h: torch.Tensor, y, mult: float = 1.0, copy: Optional[torch.Tensor] = None) -> torch.Tensor:
+        """The norm on a sublayer's output and the addition behind it, in place: h += mult * norm(y).  y [N, H] in any
+        type, or SublayerPieces, which are added up on the way; copy [N, H]: the new h in this tensor's type as well."""
+        pieces = y.as_args() if isinstance(y, SublayerPieces) else {"y": y}
+        return ops.output_norm_add(h, self.gain, self.eps, mult, copy=copy, **pieces)
 
 
 @NORMS.register("layernorm")
