@@ -74,18 +74,22 @@ def gated_unit(x: torch.Tensor, w: Dict[str, torch.Tensor], p: str) -> torch.Ten
 
 
 def choose(scores: torch.Tensor, correction: torch.Tensor, top: int, count: int, keep: int) -> Tuple[List[int], float]:
-    """One token's chosen outputs, and by how much the choice is made (in choice scores; the nearer of the last group
-    kept over the first left out and the last choice over the first eligible one left out)."""
+    """One token's chosen outputs, and how clearly they are chosen: the distance of the last group kept from the first
+    left out and of the last output chosen from the first eligible one left out, the smaller of the two, over the scores
+    that stand against each other (a choice that rounding may turn has a small one)."""
     n = scores.numel()
     c = scores + correction
     size = n // count
-    best = [float(c[g * size:(g + 1) * size].max()) for g in range(count)]
-    order = sorted(range(count), key=lambda g: (-best[g], g))
+    best = [max(range(g * size, (g + 1) * size), key=lambda e: float(c[e])) for g in range(count)]
+    order = sorted(range(count), key=lambda g: (-float(c[best[g]]), g))
     kept = set(order[:keep])
-    margin = best[order[keep - 1]] - best[order[keep]] if keep < count else math.inf
+
+    def clear(a, b):
+        return float(c[a] - c[b]) / float(scores[a] + scores[b])
+    margin = clear(best[order[keep - 1]], best[order[keep]]) if keep < count else math.inf
     eligible = sorted((e for e in range(n) if e // size in kept), key=lambda e: (-float(c[e]), e))
     if top < len(eligible):
-        margin = min(margin, float(c[eligible[top - 1]] - c[eligible[top]]))
+        margin = min(margin, clear(eligible[top - 1], eligible[top]))
     return eligible[:top], margin
 
 
@@ -98,7 +102,7 @@ def mixture(x: torch.Tensor, w: Dict[str, torch.Tensor], p: str, mlp: dict, marg
     least = []
     for t in range(x.shape[0]):
         chosen, margin = choose(scores[t], w[p + "correction"], top, int(groups["count"]), int(groups["keep"]))
-        least.append(margin * scores.shape[1])
+        least.append(margin)
         total = float(sum(scores[t, e] for e in chosen)) + 1e-20
         for e in chosen:
             weight = scores[t, e] / total * float(ro.get("scale", 1.0))
@@ -113,8 +117,8 @@ def mixture(x: torch.Tensor, w: Dict[str, torch.Tensor], p: str, mlp: dict, marg
 def forward(cfg: dict, w: Dict[str, torch.Tensor], ids: List[int], streams: Optional[list] = None,
             margins: Optional[list] = None, rounded: bool = False) -> torch.Tensor:
     """Logits [T, vocab] of one sequence from position 0.  streams: a list that receives the residual stream after
-    every layer; margins: a list that receives, per mixture, every token's margin of choice in units of the mean
-    score; rounded: every sublayer's input and result, the queries, keys, values and heads' outputs and the last norm's
+    every layer; margins: a list that receives, per mixture, every token's margin of choice (`choose`);
+    rounded: every sublayer's input and result, the queries, keys, values and heads' outputs and the last norm's
     output are rounded to bfloat16, which shows how far rounding alone moves this model's logits."""
     def r16(x):
         return x.to(torch.bfloat16).to(DT) if rounded else x
