@@ -254,6 +254,26 @@ def fedovik_pair_configs(key: str, window: int):
     return fed, lis
 
 
+def tipetar_pair_configs(key: str, window: int):
+    """(Tipetar config.json, Kigalix config.json) of equal sizes.  Tipetar: slope attention over `window` positions, every
+    second layer on the keys and values of the layer in front of it; behind every mixer sixteen experts of an eighth of
+    the dense feed-forward's size, four of twenty outputs chosen (four of them hand the input through) from two of four
+    groups, and a shared expert of a quarter of that size.  Kigalix: one residual stream, latent attention (192 + 64
+    numbers a token, every key seen) in every layer, and the same sixteen experts with four a token (no shared one)."""
+    width, layers, heads, kv, d, ff, vocab = PAIR_SIZES[key]
+    experts = {"kind": "moe", "expert": {"ff": ff // 8}, "router": {"experts": 16, "top": 4}}
+    mlp = {"kind": "moe", "expert": {"ff": ff // 8}, "shared": {"ff": ff // 4},
+           "router": {"experts": 16, "top": 4, "identity": 4, "groups": {"count": 4, "keep": 2}, "scale": 1.5}}
+    att = {"heads": heads, "kv_heads": kv, "dim": d, "vdim": d, "scale": d ** -0.5, "mask": {"size": window}}
+    tip = {"architecture": "Tipetar", "vocab": vocab, "width": width, "norm": {"eps": 1e-6}, "residual_mult": 0.7,
+           "layers": [{"type": "attention", "mixer": dict(att, **({"kv_from": i - 1} if i % 2 else {})), "mlp": mlp}
+                      for i in range(layers)], "max_positions": 32768}
+    lat = {"heads": heads, "dim": d, "rot_dim": 64, "vdim": d, "kv_rank": 192, "scale": (d + 64) ** -0.5, "rot": {"dims": 64, "base": 1e6}}
+    kig = {"architecture": "Kigalix", "vocab": vocab, "width": width, "norm": {"eps": 1e-6},
+           "layers": [{"type": "latent_attention", "mixer": lat, "mlp": experts} for _ in range(layers)], "max_positions": 32768}
+    return tip, kig
+
+
 class PairBench(Bench):
     """Bench's measurements on an engine built from any config.json."""
 
@@ -277,9 +297,9 @@ class PairBench(Bench):
 
 def design_pairs(args, design: str) -> int:
     """Prefill and decode of a second design (lisunex or gabelorn beside Qwen2, kigalix beside Gabelorn, fedovik beside
-    Lisunex) at equal sizes; one JSON line."""
+    Lisunex, tipetar beside Kigalix) at equal sizes; one JSON line."""
     title = design.capitalize()
-    beside = {"kigalix": "gabelorn", "fedovik": "lisunex"}.get(design, "qwen2")
+    beside = {"kigalix": "gabelorn", "fedovik": "lisunex", "tipetar": "kigalix"}.get(design, "qwen2")
     keys = [k.strip() for k in getattr(args, design).split(",") if k.strip()]
     for k in keys:
         if k not in PAIR_SIZES:
@@ -289,9 +309,9 @@ def design_pairs(args, design: str) -> int:
     per_req = -(-(prompt_len + args.steps + args.warmup + 32) // 16) * 16
     pool = max(batch * per_req, T + 64)
     span = {"lisunex": args.lisunex_chunk, "gabelorn": args.gabelorn_window, "kigalix": args.kigalix_streams,
-            "fedovik": args.fedovik_window}[design]
+            "fedovik": args.fedovik_window, "tipetar": args.tipetar_window}[design]
     make = {"lisunex": pair_configs, "gabelorn": gabelorn_pair_configs, "kigalix": kigalix_pair_configs,
-            "fedovik": fedovik_pair_configs}[design]
+            "fedovik": fedovik_pair_configs, "tipetar": tipetar_pair_configs}[design]
     only = getattr(args, "only", "")
     out = {}
     for k in keys:
@@ -323,7 +343,8 @@ def design_pairs(args, design: str) -> int:
         "vs_baseline": None, "dtype": {"bfloat16": "bf16", "float16": "fp16"}[args.dtype],
         "data": "synthetic (random weights N(0,0.02), uniform random token ids)",
         "config": {"model": f"{title} and {beside.capitalize()} at equal sizes", "global_batch": batch, "seq_len": prompt_len,
-                   "prefill_tokens": T, {"lisunex": "chunk", "gabelorn": "window", "kigalix": "streams", "fedovik": "window"}[design]: span,
+                   "prefill_tokens": T, {"lisunex": "chunk", "gabelorn": "window", "kigalix": "streams", "fedovik": "window",
+                                          "tipetar": "window"}[design]: span,
                    "parallelism": "1 GPU"},
         "pairs": out}), flush=True)
     return 0
@@ -389,19 +410,25 @@ def main() -> int:
                          "Lisunex at equal sizes, prefill of --prefill-tokens and decode at --batch; sizes by name, with "
                          "commas: " + ", ".join(PAIR_SIZES))
     ap.add_argument("--fedovik-window", type=int, default=1024, help="positions that the windowed attention of Fedovik sees")
+    ap.add_argument("--tipetar", default="", metavar="SIZES",
+                    help="another workload instead: the Tipetar design (slope attention in a window, every second layer on "
+                         "its neighbour's keys, a grouped mixture with identity choices and a shared expert) beside Kigalix "
+                         "(latent attention and as many experts) at equal sizes, prefill of --prefill-tokens and decode at "
+                         "--batch; sizes by name, with commas: " + ", ".join(PAIR_SIZES))
+    ap.add_argument("--tipetar-window", type=int, default=1024, help="positions that a Tipetar layer sees")
     ap.add_argument("--only", default="", metavar="MODEL",
-                    help="with --lisunex, --gabelorn, --kigalix or --fedovik: measure one model of the pair alone "
+                    help="with --lisunex, --gabelorn, --kigalix, --fedovik or --tipetar: measure one model of the pair alone "
                          "(profiling runs)")
     args = ap.parse_args()
     if args.gpus != 1 or int(os.environ.get("WORLD_SIZE", "1")) != 1:
         print("bench.py: this engine runs on one GPU; N > 1 is not measured")
         return 2
 
-    if args.lisunex or args.gabelorn or args.kigalix or args.fedovik:
+    designs = [d for d in ("lisunex", "gabelorn", "kigalix", "fedovik", "tipetar") if getattr(args, d)]
+    if designs:
         if args.dtype == "float16":
             args.dtype = "bfloat16"         # the serving dtype of these designs
-        return design_pairs(args, "lisunex" if args.lisunex else "gabelorn" if args.gabelorn else
-                            "kigalix" if args.kigalix else "fedovik")
+        return design_pairs(args, designs[0])
 
     import torch
 

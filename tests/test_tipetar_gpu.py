@@ -228,6 +228,14 @@ def test_router_forms(dtype, experts, identity, top, groups, width, with_bias):
     wts, idw = torch.full((n, top), -1.0, device=DEV), torch.full((n,), -1.0, device=DEV)
     ops.moe_route(x.to(DEV), wr.to(DEV), ids, wts, "softmax", True, 1e-20, 1.7, bias.to(DEV) if with_bias else None, groups[0],
                   groups[1], identity, idw)
+    # many tokens go four to a block, a few hundred one to a block of fewer waves: the same bits for a token
+    for rows in (300, 1030):
+        place = torch.arange(rows) % n
+        more = [torch.full((rows, top), -7, dtype=torch.int32, device=DEV), torch.full((rows, top), -1.0, device=DEV),
+                torch.full((rows,), -1.0, device=DEV)]
+        ops.moe_route(x[place].to(DEV), wr.to(DEV), more[0], more[1], "softmax", True, 1e-20, 1.7,
+                      bias.to(DEV) if with_bias else None, groups[0], groups[1], identity, more[2])
+        assert all(torch.equal(a, b[place.to(DEV)]) for a, b in zip(more, (ids, wts, idw)))
     ids, wts, idw = ids.cpu(), wts.cpu().double(), idw.cpu().double()
     scores = torch.softmax(x.double() @ wr.double().T, dim=-1)
     compared = handed = 0

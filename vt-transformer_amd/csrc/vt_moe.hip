@@ -20,22 +20,35 @@
 
 VT_DEFINE_LAST_ERROR()
 
-// a wave's dot product of a float32 row with a float32 vector in LDS, 16 bytes per lane at a time where the row allows
-__device__ __forceinline__ float wave_dot_f32(const float* __restrict__ row, const float* __restrict__ v, int K, int lane) {
-    float acc = 0.f;
+// a wave's dot products of a float32 row with TOK float32 vectors in LDS (`stride` floats apart), 16 bytes per lane at a
+// time where the row allows; a vector's sum takes its terms in the same order whatever TOK is
+template <int TOK>
+__device__ __forceinline__ void wave_dots_f32(const float* __restrict__ row, const float* __restrict__ v, int stride, int K, int lane,
+                                              float* acc) {
+#pragma unroll
+    for (int i = 0; i < TOK; ++i) acc[i] = 0.f;
     if (K % 4 == 0 && !((uintptr_t)row & 15)) {
 #pragma unroll 4
         for (int j = lane * 4; j < K; j += 256) {
             const float4 w = *(const float4*)(row + j);
-            acc = fmaf(w.x, v[j], acc);
-            acc = fmaf(w.y, v[j + 1], acc);
-            acc = fmaf(w.z, v[j + 2], acc);
-            acc = fmaf(w.w, v[j + 3], acc);
+#pragma unroll
+            for (int i = 0; i < TOK; ++i) {
+                const float4 x = *(const float4*)(v + i * stride + j);
+                acc[i] = fmaf(w.x, x.x, acc[i]);
+                acc[i] = fmaf(w.y, x.y, acc[i]);
+                acc[i] = fmaf(w.z, x.z, acc[i]);
+                acc[i] = fmaf(w.w, x.w, acc[i]);
+            }
         }
     } else {
-        for (int j = lane; j < K; j += 64) acc = fmaf(row[j], v[j], acc);
+        for (int j = lane; j < K; j += 64) {
+            const float w = row[j];
+#pragma unroll
+            for (int i = 0; i < TOK; ++i) acc[i] = fmaf(w, v[i * stride + j], acc[i]);
+        }
     }
-    return wave_sum(acc);
+#pragma unroll
+    for (int i = 0; i < TOK; ++i) acc[i] = wave_sum(acc[i]);
 }
 
 struct RouteArgs {
@@ -45,30 +58,43 @@ struct RouteArgs {
     int* ids;                   // [n][top]
     float* wts;                 // [n][top]
     float* id_wts;              // [n] or null: the weight of the chosen outputs that are no experts
-    int E, W, top, softmax, renorm, groups, keep, identity;
+    int n, E, W, top, softmax, renorm, groups, keep, identity;
     float renorm_eps, out_scale;
 };
 
-// A block of four waves per token: the token lies in LDS as float32, the waves take the experts in turn, and the
-// first wave then picks the largest scores.
-template <typename TI>
-__global__ __launch_bounds__(256) void moe_route_kernel(RouteArgs a) {
-    extern __shared__ float sh[];       // W values of the token, E scores, E choice scores, the groups' best
-    const int E = a.E, W = a.W, top = a.top;
+// A block per TOK tokens: they lie in LDS as float32, the block's waves take the router's rows in turn (a row is read once
+// for all of them), and then a wave per token picks its largest scores.  Few tokens: one to a block of sixteen waves, which
+// shortens the turns; many tokens: four to a block of four waves, which read a quarter of the router's rows.
+template <typename TI, int TOK>
+__global__ __launch_bounds__(1024) void moe_route_kernel(RouteArgs a) {
+    extern __shared__ __attribute__((aligned(16))) float sh[];      // TOK tokens of W4 floats, then per token E scores, E choice
+                                                                    // scores and the groups' best
+    const int E = a.E, W = a.W, top = a.top, W4 = (W + 3) & ~3;
+    const bool own_choice = a.correction || a.groups > 1;           // (without either, the scores themselves are chosen from)
+    const int per = E + (own_choice ? E + a.groups : 0);
     float* xs = sh;
-    float* sc = sh + W;
-    float* ch = a.correction || a.groups > 1 ? sc + E : sc;     // (without either, the scores themselves are chosen from)
-    float* gb = sc + 2 * E;
-    const int t = blockIdx.x, wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
-    const TI* xt = (const TI*)a.x + (size_t)t * W;
-    for (int j = threadIdx.x; j < W; j += 256) xs[j] = load_f32<TI>(xt, j);
-    __syncthreads();
-    for (int e = wave; e < E; e += 4) {
-        const float acc = wave_dot_f32(a.wr + (size_t)e * W, xs, W, lane);
-        if (lane == 0) sc[e] = acc;
+    const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, waves = blockDim.x >> 6;
+    const int t0 = blockIdx.x * TOK;
+#pragma unroll
+    for (int i = 0; i < TOK; ++i) {
+        const TI* xt = (const TI*)a.x + (size_t)(t0 + i) * W;
+        for (int j = threadIdx.x; j < W; j += blockDim.x) xs[i * W4 + j] = t0 + i < a.n ? load_f32<TI>(xt, j) : 0.f;
     }
     __syncthreads();
-    if (wave != 0) return;
+    for (int e = wave; e < E; e += waves) {
+        float acc[TOK];
+        wave_dots_f32<TOK>(a.wr + (size_t)e * W, xs, W4, W, lane, acc);
+        if (lane == 0) {
+#pragma unroll
+            for (int i = 0; i < TOK; ++i) sh[TOK * W4 + i * per + e] = acc[i];
+        }
+    }
+    __syncthreads();
+    const int t = t0 + wave;
+    if (wave >= TOK || t >= a.n) return;
+    float* sc = sh + TOK * W4 + wave * per;
+    float* ch = own_choice ? sc + E : sc;
+    float* gb = sc + 2 * E;
     if (a.softmax) {
         float m = -INFINITY;
         for (int e = lane; e < E; e += 64) m = fmaxf(m, sc[e]);
@@ -105,17 +131,20 @@ __global__ __launch_bounds__(256) void moe_route_kernel(RouteArgs a) {
     }
     float total = 0.f, id_total = 0.f;
     for (int k = 0; k < top; ++k) {
-        float best = -INFINITY;
+        float mine = -INFINITY;
         int at = 0x7fffffff;
         for (int e = lane; e < E; e += 64) {
             const float v = ch[e];
-            if (v > best) { best = v; at = e; }
+            if (v > mine) { mine = v; at = e; }
         }
+        const float best = wave_max(mine);
+        if (mine != best) at = 0x7fffffff;
+        if (E <= 64) {              // a lane has one output: the lowest lane has the lowest index
+            const unsigned long long who = __ballot(at != 0x7fffffff);
+            at = who ? __ffsll(who) - 1 : 0x7fffffff;
+        } else {
 #pragma unroll
-        for (int o = 32; o > 0; o >>= 1) {
-            const float ob = __shfl_xor(best, o, 64);
-            const int oa = __shfl_xor(at, o, 64);
-            if (ob > best || (ob == best && oa < at)) { best = ob; at = oa; }
+            for (int o = 32; o > 0; o >>= 1) at = min(at, __shfl_xor(at, o, 64));
         }
         if (at == 0x7fffffff) at = k < E ? k : 0;     // scores that are no numbers: some expert all the same
         const float s = sc[at];
@@ -145,14 +174,20 @@ extern "C" int vt_moe_route(const void* x, int dtype, const float* wr, int* ids,
     VT_REQUIRE(groups >= 1 && E % groups == 0 && keep >= 1 && keep <= groups && top <= keep * (E / groups),
                "vt_moe_route: %d of %d groups of %d experts, %d chosen", keep, groups, E, top);
     VT_REQUIRE(identity >= 0 && identity < E && (identity == 0 || id_wts), "vt_moe_route: %d of %d outputs without an expert", identity, E);
-    const size_t floats = (size_t)W + E + (correction || groups > 1 ? E + groups : 0);
+    VT_REQUIRE(dtype == VT_F32 || dtype == VT_BF16, "vt_moe_route: unknown dtype %d", dtype);
+    const size_t floats = (((size_t)W + 3) & ~(size_t)3) + E + (correction || groups > 1 ? E + groups : 0);
     VT_REQUIRE(floats <= 16000, "vt_moe_route: %d experts and a width of %d (the scores and the token together up to 16000 floats)", E, W);
     if (n == 0) return 0;
-    RouteArgs a = {x, wr, correction, ids, wts, id_wts, E, W, top, softmax, renorm, groups, keep, identity, renorm_eps, out_scale};
-    const size_t lds = floats * sizeof(float);
-    if (dtype == VT_F32) moe_route_kernel<float><<<n, 256, lds, stream>>>(a);
-    else if (dtype == VT_BF16) moe_route_kernel<bf16_t><<<n, 256, lds, stream>>>(a);
-    else return vt_fail("vt_moe_route: unknown dtype %d", dtype);
+    RouteArgs a = {x, wr, correction, ids, wts, id_wts, n, E, W, top, softmax, renorm, groups, keep, identity, renorm_eps, out_scale};
+    const bool four = n >= 1024 && 4 * floats <= 16000;
+    const int threads = n <= 256 ? 1024 : 256;
+    if (dtype == VT_F32) {
+        if (four) moe_route_kernel<float, 4><<<(n + 3) / 4, 256, 4 * floats * sizeof(float), stream>>>(a);
+        else moe_route_kernel<float, 1><<<n, threads, floats * sizeof(float), stream>>>(a);
+    } else {
+        if (four) moe_route_kernel<bf16_t, 4><<<(n + 3) / 4, 256, 4 * floats * sizeof(float), stream>>>(a);
+        else moe_route_kernel<bf16_t, 1><<<n, threads, floats * sizeof(float), stream>>>(a);
+    }
     VT_CHECK_LAUNCH("vt_moe_route");
     return 0;
 }

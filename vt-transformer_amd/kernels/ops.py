@@ -1021,12 +1021,17 @@ def attention_masked_mfma(q: torch.Tensor, k_pages: torch.Tensor, v_pages: torch
     return out
 
 
-def attention_masked_decode_splits(n: int, n_heads: int, n_kv: int, max_len: int) -> int:
+def attention_masked_decode_splits(n: int, n_heads: int, n_kv: int, max_len: int, reach: int = 0) -> int:
     """Into how many blocks of four waves a decoding step's keys are dealt per (token, group of heads): enough to give
-    every compute unit a few waves, no more than there are turns of 32 keys in the longest sequence.  It depends on
-    the number of tokens and the engine's limits alone, so that a recorded step can be replayed."""
+    every compute unit a few waves, no more than there are turns of 32 keys in the longest sequence, or in the `reach`
+    positions that a mask leaves of it (0: all).  It depends on the number of tokens, the mask and the engine's limits
+    alone, so that a recorded step can be replayed."""
     tiles = max(1, n) * n_kv * (-(-(n_heads // n_kv) // 16))
-    return int(max(1, min(-(-512 // tiles), max(1, max_len // 128), 16)))
+    most = max(1, max_len // 128)
+    if reach > 0:
+        turns = (reach + 14) // 32 + 1          # (the first turn starts at a multiple of 16)
+        most = min(most, -(-turns // 4))
+    return int(max(1, min(-(-512 // tiles), most, 16)))
 
 
 def attention_masked_decode(q: torch.Tensor, k_pages: torch.Tensor, v_pages: torch.Tensor, positions: torch.Tensor,

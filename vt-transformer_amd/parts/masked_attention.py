@@ -87,7 +87,7 @@ def run_masked_attention(rt: Runtime, ctx, cache, q: torch.Tensor, out: torch.Te
               sigmoid_weights=sigmoid_weights, gate_wide=gate_wide)
     if cores and ctx.single_token:
         n = q.shape[0]
-        splits = ops.attention_masked_decode_splits(n, nh, nkv, ctx.n_positions)
+        splits = ops.attention_masked_decode_splits(n, nh, nkv, ctx.n_positions, min([w for w in (window, chunk) if w > 0], default=0))
         part = rt.buffer("mattn.decode_parts", (ops.attention_masked_decode_scratch(n, nh, nkv, dv, splits),), torch.float32)
         return ops.attention_masked_decode(q, cache["k"], cache["v"], ctx.positions, ctx.tok_entry, cache.block_table, out,
                                            part, splits, nh, nkv, d, dv, scale, softcap, window, chunk, **kw)
