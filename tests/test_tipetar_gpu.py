@@ -24,12 +24,12 @@ CUTS = [(0, 20), (20, 21), (21, 23), (23, 70), (70, 71), (71, 83)]
 
 @pytest.fixture(scope="module")
 def folders(tmp_path_factory):
-    """Every configuration twice: as it is, and with fixed routes (what bfloat16 compares)."""
+    """Every configuration twice: as it is, and with fixed routes (what the 16-bit types compare)."""
     root = tmp_path_factory.mktemp("tipetar")
     out = {}
     for i, (k, cfg) in enumerate(CONFIGS.items()):
         out[k, "float32"] = write_model(copy.deepcopy(cfg), str(root / k), seed=41 + i, idle=k == "A")
-        out[k, "bfloat16"] = write_model(copy.deepcopy(cfg), str(root / (k + "f")), seed=51 + i, fixed_routes=True)
+        out[k, "bfloat16"] = out[k, "float16"] = write_model(copy.deepcopy(cfg), str(root / (k + "f")), seed=51 + i, fixed_routes=True)
     return out
 
 
@@ -432,8 +432,7 @@ def test_blocks_of_other_kinds_around_this_one(tmp_path):
 LENGTHS = [61, 1, 23, 90, 2, 47]
 
 
-@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
-@pytest.mark.parametrize("name", ["A", "B", "C", "D"])
+@pytest.mark.parametrize("name,dtype", [(n, d) for n in "ABCD" for d in ("float32", "bfloat16")] + [("A", "float16"), ("D", "float16")])
 def test_schedules(folders, name, dtype):
     """Whole prompts; most of a prompt and then its last tokens one by one; portions of changing sizes down to two
     tokens; unequal requests side by side with three slots and few pages, so that both are used again."""

@@ -13,7 +13,7 @@ import torch
 import plain_tipetar as pt
 
 # root mean square of a row's error (its mean taken off) over the root mean square of the row's logits (theirs too)
-TOL = {"float32": 3e-5, "bfloat16": 2e-2}
+TOL = {"float32": 3e-5, "bfloat16": 2e-2, "float16": 4e-3}
 # Rounding may send a token whose choice of experts is nearly a tie to other experts than the plain implementation
 # sends it to.  Two measures: models that are compared in bfloat16 have "fixed routes" (make_weights), whose routers read
 # numbers that bfloat16 holds exactly, so that their logits are float32's in both dtypes; and a position that a token can
@@ -138,7 +138,7 @@ def _in_doubt(cfg: dict, least: Optional[np.ndarray], n: int) -> np.ndarray:
 def check_logits(model_dir: str, reqs: Dict[str, List[int]], steps: List[dict], got: Dict[int, np.ndarray], dtype: str,
                  cache: dict = None, least_compared: float = 0.9) -> float:
     """Every wanted row against the plain implementation's logits at that place; raises at the first row beyond
-    its limit, naming step, request and position.  In bfloat16 a position's limit is the tolerance, or three times what
+    its limit, naming step, request and position.  In 16 bits a position's limit is the tolerance, or three times what
     rounding alone does to it where that is more.  Returns the worst error."""
     cfg, w = pt.read_folder(model_dir)
     cache = cache if cache is not None else {}
@@ -149,8 +149,9 @@ def check_logits(model_dir: str, reqs: Dict[str, List[int]], steps: List[dict], 
             margins = []
             logits = pt.forward(cfg, w, toks, margins=margins).numpy()
             least = torch.stack(margins).min(dim=0).values.numpy() if margins else None
+            # (float16 rounds eight times finer than bfloat16)
             moved = row_errors(pt.forward(cfg, w, toks, rounded=True).numpy(), logits)
-            cache[key] = (logits, least, np.maximum(TOL["bfloat16"], 3.0 * moved))
+            cache[key] = (logits, least, 3.0 * moved)
         ref[rid], least, limit[rid] = cache[key]
         doubt[rid] = _in_doubt(cfg, least, len(toks))
     pos = {r: 0 for r in reqs}
@@ -169,7 +170,9 @@ def check_logits(model_dir: str, reqs: Dict[str, List[int]], steps: List[dict], 
                     skipped += 1
                     continue
                 err = float(row_errors(gl[None], r[None])[0])
-                lim = TOL["float32"] if dtype == "float32" else float(limit[e["id"]][p])
+                lim = TOL[dtype]
+                if dtype != "float32":
+                    lim = max(lim, float(limit[e["id"]][p]) / (8.0 if dtype == "float16" else 1.0))
                 assert err < lim, (f"step {s['step']} request {e['id']} position {p} "
                                    f"(portion starts at {pos[e['id']]}): error {err:.3e} > {lim:.1e}")
                 worst = max(worst, err)
