@@ -14,7 +14,7 @@ Shaped after the reference's PageTable and CacheManager
 Differences: the block table has one entry per page, not per token; layers
 with different needs (all keys, or a window of them) form groups with pools
 and tables of their own; a page that a window has passed is given back at
-once; and there is no prefix tree, so a finished request returns everything
+once (a window may keep a sequence's first tokens: their pages stay); and there is no prefix tree, so a finished request returns everything
 (the reference keeps prefixes in a radix tree that nothing ever evicts,
 vt_cache.hpp:121-166, 264-269).
 """
@@ -95,11 +95,13 @@ class SlotPool:
 
 @dataclass
 class GroupSpec:
-    """Layers with the same need: `window` 0 keeps every key; W > 0 keeps the last W."""
+    """Layers with the same need: `window` 0 keeps every key; W > 0 keeps the last W and a sequence's first
+    `keep_first`."""
 
     key: Hashable
     window: int
     num_pages: int
+    keep_first: int = 0
 
 
 @dataclass
@@ -158,16 +160,22 @@ class CacheManager:
             return 0
         return max(0, (length - w + 1)) // self.page_size
 
+    def _kept_blocks(self, gi: int) -> int:
+        """Blocks that hold tokens which stay whatever the window has passed: the leading ones."""
+        g = self.groups[gi]
+        return -(-g.keep_first // self.page_size) if g.window > 0 else 0
+
     def max_held_pages(self, gi: int, portion: int) -> int:
         """The most pages of group gi that one request can hold at a time when no step brings more than `portion`
         of its tokens: every page for a group that keeps all keys; for a group with a window, the pages of the
-        window and of one portion (and one more: neither needs to start at a page's edge)."""
+        window and of one portion (and one more: neither needs to start at a page's edge) and those of the first
+        tokens that it keeps."""
         ps = self.page_size
         whole = -(-self.max_seq_len // ps)
         w = self.groups[gi].window
         if w <= 0:
             return whole
-        return min(whole, -(-(w + max(1, int(portion))) // ps) + 1)
+        return min(whole, -(-(w + max(1, int(portion))) // ps) + 1 + self._kept_blocks(gi))
 
     def pages_needed(self, rp: RequestPages, new_len: int, portion: Optional[int] = None) -> List[int]:
         """Per group, how many pages `reserve` would have to take for the request to hold new_len tokens after
@@ -231,10 +239,11 @@ class CacheManager:
         rp.fresh = False
         for gi, table in enumerate(rp.tables):
             dead_before = min(self._first_live_block(gi, new_len), len(table))
-            gone = [table[b] for b in range(dead_before) if table[b] != NO_PAGE]
+            kept = self._kept_blocks(gi)
+            gone = [table[b] for b in range(kept, dead_before) if table[b] != NO_PAGE]
             if gone:
                 self.pools[gi].free(gone)
-                for b in range(dead_before):
+                for b in range(kept, dead_before):
                     table[b] = NO_PAGE
 
     # -- queries ----------------------------------------------------------

@@ -37,7 +37,7 @@ class LayerCache:
 def group_pages(needs: List[CacheNeed], page_bytes: List[int], page_size: int, max_requests: int, max_seq_len: int,
                 max_portion: int, kv_bytes: int) -> List[int]:
     """Pages per group under a budget in bytes for all of them.  A group with a window never holds more of a
-    request than its window and one portion (CacheManager.max_held_pages), so it gets pages for that, for every
+    request than its window, one portion and the first tokens that it keeps (CacheManager.max_held_pages), so it gets pages for that, for every
     request that may run, and no more; what is left of the budget goes to the groups that keep every key, which all
     hold the same tokens and so get the same number of pages: budget // (bytes of one page of each of them together),
     as the reference sizes its one pool (vt-transformer/models/qwen3-0.6b/init.vt:109-113:
@@ -49,7 +49,8 @@ def group_pages(needs: List[CacheNeed], page_bytes: List[int], page_size: int, m
         if need.window > 0:
             # (what a request holds at most, and the page of head-room per running request that the scheduler keeps
             # free when it admits another)
-            per_request = min(whole, -(-(need.window + max(1, max_portion)) // page_size) + 1) + 1
+            kept = -(-need.keep_first // page_size)
+            per_request = min(whole, -(-(need.window + max(1, max_portion)) // page_size) + 1 + kept) + 1
             pages[g] = max(1, min(max_requests * per_request, left // max(1, page_bytes[g])))
             left -= pages[g] * page_bytes[g]
     unbounded = [g for g, need in enumerate(needs) if need.window <= 0]
@@ -90,12 +91,14 @@ class CacheStorage:
                     raise ValueError(f"schedule entry {i} cannot read the cache of entry {e.cache_from}: "
                                      f"their pages differ")
         # A cache that further entries read keeps a token until the last of its readers has passed it: an entry's need
-        # has the widest window among its own and its readers' (0 if one of them sees every token).
+        # has the widest window among its own and its readers' (0 if one of them sees every token), and keeps as many of
+        # the first tokens as the one that keeps the most.
         for i, e in enumerate(schedule):
             if e.cache_from is not None:
                 own, reach = needs[e.cache_from], needs[i].window
                 keep = max(own.window, reach) if own.window > 0 and reach > 0 else 0
-                needs[e.cache_from] = replace(own, window=keep)
+                first = max(own.keep_first, needs[i].keep_first) if keep > 0 else 0
+                needs[e.cache_from] = replace(own, window=keep, keep_first=first)
         # groups of entries with their own cache and equal needs
         keys: List = []
         self.group_needs: List[CacheNeed] = []
@@ -130,7 +133,7 @@ class CacheStorage:
                 raise ValueError("the cache needs a size: pool_tokens or kv_bytes")
             pages = [max(1, -(-int(pool_tokens) // self.page_size))] * len(self.group_needs)
         self.group_pages = pages
-        self.manager = CacheManager([GroupSpec(k, need.window, n) for k, need, n in zip(keys, self.group_needs, pages)],
+        self.manager = CacheManager([GroupSpec(k, need.window, n, need.keep_first) for k, need, n in zip(keys, self.group_needs, pages)],
                                     self.page_size, max_requests, max_seq_len)
         # per group and page tensor: [layer][page] + the tensor's page shape
         self.pages: List[Dict[str, torch.Tensor]] = []

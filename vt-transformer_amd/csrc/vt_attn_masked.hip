@@ -12,6 +12,7 @@
 //                   not on how its request was cut into steps or what else is in the batch.
 //                   score = cap * tanh(scale * q.k / cap) (cap 0: none); key j is seen from position i if j <= i,
 //                   i - j < window (window 0: no bound) and j >= floor(i / chunk) * chunk (chunk 0: no bound);
+//                   keep_first (with a window): the keys j < keep_first are seen from every later position as well;
 //                   out = softmax(score) V * sigmoid(gate[token][head]) (no gate pointer: no gate).
 //                   With `slopes`, slopes[head] * (i - j) is taken off the score of key j (behind the cap); with
 //                   `sink`, exp(sink[head]) joins the softmax's denominator and nothing else: a key that holds no
@@ -320,7 +321,7 @@ struct MaskedArgs {
     long long ldg;
     int sigmoid_weights;    // 1: weight = sigmoid(score), not normalized
     int gate_wide;          // 1: gate[t * ldg + h * Dv + d]
-    int H, G, D, Dv, page_size, max_blocks, num_pages, window, chunk;
+    int H, G, D, Dv, page_size, max_blocks, num_pages, window, chunk, keep_first;
     float scale, cap;
 };
 
@@ -341,6 +342,7 @@ __global__ __launch_bounds__(KEYS) void attn_masked_kernel(MaskedArgs a) {
     const int* bt = a.block_table + (size_t)a.tok_entry[t] * a.max_blocks;
     int lo = a.chunk > 0 ? (pos / a.chunk) * a.chunk : 0;
     if (a.window > 0) lo = max(lo, pos - a.window + 1);
+    const int keep = min(a.keep_first, lo);     // seen: [0, keep) and [lo, pos]
     const TC* kp = (const TC*)a.k_pages;
     const TC* vp = (const TC*)a.v_pages;
     const float slope = a.slopes ? a.slopes[h] : 0.f;
@@ -358,9 +360,10 @@ __global__ __launch_bounds__(KEYS) void attn_masked_kernel(MaskedArgs a) {
 
     float m = -INFINITY, l = 0.f, acc = 0.f;
     float acc_w[3] = {0.f, 0.f, 0.f};        // columns tid + KEYS, tid + 2 KEYS, tid + 3 KEYS of a wide head
-    for (int c0 = (lo / KEYS) * KEYS; c0 <= pos; c0 += KEYS) {
+    const int c_lo = (lo / KEYS) * KEYS;
+    for (int c0 = keep > 0 ? 0 : c_lo; c0 <= pos; c0 = c0 + KEYS >= keep ? max(c0 + KEYS, c_lo) : c0 + KEYS) {
         const int j = c0 + tid;
-        const bool valid = j >= lo && j <= pos;
+        const bool valid = (j >= lo || j < keep) && j <= pos;
         float s = -INFINITY;
         if (valid) {
             const int blk = j / ps;
@@ -397,7 +400,7 @@ __global__ __launch_bounds__(KEYS) void attn_masked_kernel(MaskedArgs a) {
         if (pv_active) {
             for (int jj = g_own; jj < KEYS; jj += Gv) {
                 const int jk = c0 + jj;
-                if (jk < lo || jk > pos) continue;
+                if ((jk < lo && jk >= keep) || jk > pos) continue;
                 const int blk = jk / ps;
                 const int pg = bt[blk];
                 if (pg < 0 || pg >= a.num_pages) continue;
@@ -412,7 +415,7 @@ __global__ __launch_bounds__(KEYS) void attn_masked_kernel(MaskedArgs a) {
                 float pw = 0.f;
                 for (int jj = 0; jj < KEYS; ++jj) {
                     const int jk = c0 + jj;
-                    if (jk < lo || jk > pos) continue;
+                    if ((jk < lo && jk >= keep) || jk > pos) continue;
                     const int blk = jk / ps;
                     const int pg = bt[blk];
                     if (pg < 0 || pg >= a.num_pages) continue;
@@ -460,7 +463,7 @@ __global__ __launch_bounds__(KEYS) void attn_masked_kernel(MaskedArgs a) {
 extern "C" int vt_attn_masked(const void* q, const void* k_pages, const void* v_pages, int dtype, const int* positions,
                               const int* tok_entry, const int* block_table, const void* gate, int gate_dtype,
                               long long ldg, void* out, int n, int H, int G, int D, int Dv, int page_size,
-                              int max_blocks, int num_pages, int window, int chunk, float scale, float cap,
+                              int max_blocks, int num_pages, int window, int chunk, int keep_first, float scale, float cap,
                               const float* sink, const float* slopes, const float* dist_r1, const float* dist_r2,
                               const float* score_shift, int sigmoid_weights, int gate_wide, hipStream_t stream) {
     VT_REQUIRE(n >= 0 && H > 0 && G > 0 && H % G == 0, "vt_attn_masked: bad heads %d/%d", H, G);
@@ -471,12 +474,14 @@ extern "C" int vt_attn_masked(const void* q, const void* k_pages, const void* v_
     VT_REQUIRE(page_size > 0 && max_blocks > 0 && num_pages > 0, "vt_attn_masked: bad cache sizes");
     VT_REQUIRE(H <= 65535, "vt_attn_masked: too many heads (%d)", H);
     VT_REQUIRE(window >= 0 && chunk >= 0 && cap >= 0.f, "vt_attn_masked: bad mask or cap");
+    VT_REQUIRE(keep_first >= 0 && (keep_first == 0 || (window > 0 && chunk == 0)), "vt_attn_masked: %d first keys kept beside window %d, chunk %d",
+               keep_first, window, chunk);
     if (n == 0) return 0;
     MaskedArgs a;
     a.q = q; a.k_pages = k_pages; a.v_pages = v_pages; a.positions = positions; a.tok_entry = tok_entry;
     a.block_table = block_table; a.gate = gate; a.out = out; a.ldg = ldg; a.H = H; a.G = G; a.D = D; a.Dv = Dv;
     a.page_size = page_size; a.max_blocks = max_blocks; a.num_pages = num_pages; a.window = window; a.chunk = chunk;
-    a.scale = scale; a.cap = cap; a.sink = sink; a.slopes = slopes; a.dist_r1 = dist_r1; a.dist_r2 = dist_r2;
+    a.keep_first = keep_first; a.scale = scale; a.cap = cap; a.sink = sink; a.slopes = slopes; a.dist_r1 = dist_r1; a.dist_r2 = dist_r2;
     a.score_shift = score_shift; a.sigmoid_weights = sigmoid_weights; a.gate_wide = gate_wide;
     const size_t shmem = (size_t)(D + 2 * KEYS) * sizeof(float);
     const dim3 grid(n, H);

@@ -16,7 +16,9 @@
 // `dist_r1`, `dist_r2`: r1[head] * ln(1 + r2[head] * (position - key index)) is taken off every score (base 2:
 // r1 * log2(1 + r2 d), the hardware's logarithm); `score_shift`: a number per head added to every score;
 // sigmoid_weights: the weight of a seen key is sigmoid(score) = 1 / (1 + 2^-score'), nothing is normalized;
-// gate_wide: one gate logit per output element, gate[token][head * Dv + d], instead of one per head.
+// gate_wide: one gate logit per output element, gate[token][head * Dv + d], instead of one per head; keep_first: beside
+// the window, the keys of the sequence's first positions are seen from everywhere (the turns that hold them are walked
+// first, and what lies between them and the window is left out: KeyTurns).
 #include "vt_common.h"
 #include <math.h>
 
@@ -46,8 +48,24 @@ struct MfmaArgs {
     const float* score_shift;   // [H] or null
     bf16_t* out;            // [n][H][Dv]
     long long ldg;
-    int n_tiles, H, G, page_size, max_blocks, num_pages, window, chunk, gate_f32, sigmoid_weights, gate_wide;
+    int n_tiles, H, G, page_size, max_blocks, num_pages, window, chunk, keep_first, gate_f32, sigmoid_weights, gate_wide;
     float scale, cap;
+};
+
+// The turns of 32 keys that hold what is seen: from the turn of `lo` on, and in front of that the turns of the first
+// `keep` keys, which never overlap the others; where the two meet there is one walk from 0.
+struct KeyTurns {
+    int first, kept, start;     // the walk begins at `first`; from `kept` (0: no jump) it goes on at `start`
+    __device__ __forceinline__ KeyTurns(int lo, int keep) {
+        start = (lo / 16) * 16;
+        kept = (keep + 31) / 32 * 32;
+        if (keep > 0 && kept >= start) start = kept = 0;
+        first = kept > 0 ? 0 : start;
+    }
+    __device__ __forceinline__ int next(int kt) const { return kt + 32 == kept ? start : kt + 32; }
+    // the i-th turn, and how many there are up to position pos
+    __device__ __forceinline__ int at(int i) const { return 32 * i < kept ? 32 * i : start + 32 * i - kept; }
+    __device__ __forceinline__ int count(int pos) const { return kept / 32 + (pos - start) / 32 + 1; }
 };
 
 // what the score's optional forms take off or add, in the base-2 domain: key j seen from position pos
@@ -150,11 +168,13 @@ __global__ __launch_bounds__(256) void attn_masked_mfma_kernel(MfmaArgs a) {
 #pragma unroll
         for (int v = 0; v < NV; ++v) vd[v] = load4(vp + (size_t)v * 16 * ps);
     };
-    const int kt0 = (lo / 16) * 16;
+    const KeyTurns turns(lo, a.keep_first);
+    const int kt0 = turns.first;
     fetch(kt0, page_of(kt0), kn[0], vn[0], ok_next[0]);
     fetch(kt0 + 16, page_of(kt0 + 16), kn[1], vn[1], ok_next[1]);
-    int pg_a = page_of(kt0 + 32), pg_b = page_of(kt0 + 48);
-    for (int kt = kt0; kt <= pos_last; kt += 32) {
+    int pg_a = page_of(turns.next(kt0)), pg_b = page_of(turns.next(kt0) + 16);
+    for (int kt = kt0, kt_next; kt <= pos_last; kt = kt_next) {
+        kt_next = turns.next(kt);
 #pragma unroll
         for (int u = 0; u < 2; ++u) {
 #pragma unroll
@@ -163,11 +183,11 @@ __global__ __launch_bounds__(256) void attn_masked_mfma_kernel(MfmaArgs a) {
             for (int v = 0; v < NV; ++v) vf[u][v] = vn[u][v];
             ok_now[u] = ok_next[u];
         }
-        if (kt + 32 <= pos_last) {
-            fetch(kt + 32, pg_a, kn[0], vn[0], ok_next[0]);
-            fetch(kt + 48, pg_b, kn[1], vn[1], ok_next[1]);
-            pg_a = page_of(kt + 64);
-            pg_b = page_of(kt + 80);
+        if (kt_next <= pos_last) {
+            fetch(kt_next, pg_a, kn[0], vn[0], ok_next[0]);
+            fetch(kt_next + 16, pg_b, kn[1], vn[1], ok_next[1]);
+            pg_a = page_of(turns.next(kt_next));
+            pg_b = page_of(turns.next(kt_next) + 16);
         }
         f32x4 s0 = {0.f, 0.f, 0.f, 0.f}, s1 = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
@@ -191,12 +211,12 @@ __global__ __launch_bounds__(256) void attn_masked_mfma_kernel(MfmaArgs a) {
             for (int i = 0; i < 8; ++i) sc[i] = forms.apply(sc[i], pos, kt + (i < 4 ? 0 : 16) + grp * 4 + (i & 3));
         }
         // a turn that every row sees whole needs no mask
-        const bool whole = kt + 31 <= pos_first && kt >= lo_last && ok_now[0] && ok_now[1];
+        const bool whole = kt + 31 <= pos_first && (kt >= lo_last || kt + 31 < a.keep_first) && ok_now[0] && ok_now[1];
         if (!whole) {
 #pragma unroll
             for (int i = 0; i < 8; ++i) {
                 const int j = kt + (i < 4 ? 0 : 16) + grp * 4 + (i & 3);
-                const bool seen = row_ok && j <= pos && j >= lo_r;
+                const bool seen = row_ok && j <= pos && (j >= lo_r || j < a.keep_first);
                 // (a missing page must show, not pass as a masked key)
                 sc[i] = seen ? (ok_now[i >> 2] ? sc[i] : nan) : -INFINITY;
             }
@@ -379,18 +399,20 @@ __global__ __launch_bounds__(256) void attn_masked_mfma_shared_kernel(MfmaArgs a
         }
     };
 
-    const int kt0 = (lo / 16) * 16;
+    const KeyTurns turns(lo, a.keep_first);
+    const int kt0 = turns.first;
     fetch(kt0, page_of(kt0), page_of(kt0 + 16));
-    int pg_a = page_of(kt0 + 32), pg_b = page_of(kt0 + 48);
+    int pg_a = page_of(turns.next(kt0)), pg_b = page_of(turns.next(kt0) + 16);
     int b = 0;
-    for (int kt = kt0; kt <= pos_last; kt += 32) {
+    for (int kt = kt0, kt_next; kt <= pos_last; kt = kt_next) {
+        kt_next = turns.next(kt);
         to_lds(b);
         ok_now[0] = ok_next[0];
         ok_now[1] = ok_next[1];
-        if (kt + 32 <= pos_last) {
-            fetch(kt + 32, pg_a, pg_b);
-            pg_a = page_of(kt + 64);
-            pg_b = page_of(kt + 80);
+        if (kt_next <= pos_last) {
+            fetch(kt_next, pg_a, pg_b);
+            pg_a = page_of(turns.next(kt_next));
+            pg_b = page_of(turns.next(kt_next) + 16);
         }
         __syncthreads();
         f32x4 s0 = {0.f, 0.f, 0.f, 0.f}, s1 = {0.f, 0.f, 0.f, 0.f};
@@ -421,12 +443,12 @@ __global__ __launch_bounds__(256) void attn_masked_mfma_shared_kernel(MfmaArgs a
 #pragma unroll
             for (int i = 0; i < 8; ++i) sc[i] = forms.apply(sc[i], pos, kt + (i < 4 ? 0 : 16) + grp * 4 + (i & 3));
         }
-        const bool whole = kt + 31 <= pos_first && kt >= lo_last && ok_now[0] && ok_now[1];
+        const bool whole = kt + 31 <= pos_first && (kt >= lo_last || kt + 31 < a.keep_first) && ok_now[0] && ok_now[1];
         if (!whole) {
 #pragma unroll
             for (int i = 0; i < 8; ++i) {
                 const int j = kt + (i < 4 ? 0 : 16) + grp * 4 + (i & 3);
-                const bool seen = row_ok && j <= pos && j >= lo_r;
+                const bool seen = row_ok && j <= pos && (j >= lo_r || j < a.keep_first);
                 sc[i] = seen ? (ok_now[i >> 2] ? sc[i] : nan) : -INFINITY;
             }
         }
@@ -519,7 +541,7 @@ struct DecodeArgs {
     float* part;
     bf16_t* out;            // [n][H][DV]
     long long ldg;
-    int n, H, G, HT, P, page_size, max_blocks, num_pages, window, chunk, gate_f32, sigmoid_weights, gate_wide;
+    int n, H, G, HT, P, page_size, max_blocks, num_pages, window, chunk, keep_first, gate_f32, sigmoid_weights, gate_wide;
     float scale, cap;
 };
 #define DEC_ROW (VT_VALUE_DIM + 4)
@@ -539,8 +561,8 @@ __global__ __launch_bounds__(256) void attn_masked_decode_kernel(DecodeArgs a) {
     const int ps = a.page_size;
     int lo = a.chunk > 0 ? (pos / a.chunk) * a.chunk : 0;
     if (a.window > 0) lo = max(lo, pos - a.window + 1);
-    const int kt0 = (lo / 16) * 16;
-    const int turns = (pos - kt0) / 32 + 1;
+    const KeyTurns walk(lo, a.keep_first);
+    const int turns = walk.count(pos);
 
     vt_lowp4_t qf[NK];
     {
@@ -564,7 +586,7 @@ __global__ __launch_bounds__(256) void attn_masked_decode_kernel(DecodeArgs a) {
     const bool sig = a.sigmoid_weights != 0;
 
     for (int turn = p; turn < turns; turn += a.P) {
-        const int kt = kt0 + turn * 32;
+        const int kt = walk.at(turn);
         vt_lowp4_t kf[2][NK], vf[2][NV];
         bool ok[2];
 #pragma unroll
@@ -600,7 +622,7 @@ __global__ __launch_bounds__(256) void attn_masked_decode_kernel(DecodeArgs a) {
             }
             const int j = kt + (i < 4 ? 0 : 16) + grp * 4 + (i & 3);
             if (forms_on) sc[i] = forms.apply(sc[i], pos, j);
-            const bool seen = row_ok && j <= pos && j >= lo;
+            const bool seen = row_ok && j <= pos && (j >= lo || j < a.keep_first);
             // (a missing page must show, not pass as a masked key)
             sc[i] = seen ? (ok[i >> 2] ? sc[i] : nan) : -INFINITY;
         }
@@ -699,7 +721,7 @@ extern "C" int vt_attn_masked_decode(const void* q, const void* k_pages, const v
                                      const int* tok_entry, const int* block_table, const void* gate, int gate_dtype,
                                      long long ldg, void* out, float* part, long long part_floats, int splits, int n,
                                      int H, int G, int D, int Dv, int page_size, int max_blocks, int num_pages, int window,
-                                     int chunk, float scale, float cap, const float* sink, const float* slopes,
+                                     int chunk, int keep_first, float scale, float cap, const float* sink, const float* slopes,
                                      const float* dist_r1, const float* dist_r2, const float* score_shift,
                                      int sigmoid_weights, int gate_wide, hipStream_t stream) {
     VT_REQUIRE((dist_r1 == nullptr) == (dist_r2 == nullptr), "vt_attn_masked_decode: the distance bias takes both of its numbers");
@@ -711,6 +733,8 @@ extern "C" int vt_attn_masked_decode(const void* q, const void* k_pages, const v
     VT_REQUIRE(page_size > 0 && page_size % 16 == 0 && max_blocks > 0 && num_pages > 0,
                "vt_attn_masked_decode: pages of %d keys (a multiple of 16)", page_size);
     VT_REQUIRE(window >= 0 && chunk >= 0 && cap >= 0.f, "vt_attn_masked_decode: bad mask or cap");
+    VT_REQUIRE(keep_first >= 0 && (keep_first == 0 || (window > 0 && chunk == 0)),
+               "vt_attn_masked_decode: %d first keys kept beside window %d, chunk %d", keep_first, window, chunk);
     VT_REQUIRE(splits >= 1 && splits <= 64, "vt_attn_masked_decode: %d splits (1 to 64)", splits);
     VT_REQUIRE(!gate || gate_dtype == VT_F32 || gate_dtype == VT_BF16, "vt_attn_masked_decode: gate dtype %d", gate_dtype);
     if (n == 0) return 0;
@@ -723,8 +747,8 @@ extern "C" int vt_attn_masked_decode(const void* q, const void* k_pages, const v
     a.q = (const bf16_t*)q; a.k_pages = (const bf16_t*)k_pages; a.v_pages = (const bf16_t*)v_pages; a.positions = positions;
     a.tok_entry = tok_entry; a.block_table = block_table; a.sink = sink; a.slopes = slopes; a.gate = gate; a.part = part;
     a.out = (bf16_t*)out; a.ldg = ldg; a.n = n; a.H = H; a.G = G; a.HT = HT; a.P = 4 * splits; a.page_size = page_size;
-    a.max_blocks = max_blocks; a.num_pages = num_pages; a.window = window; a.chunk = chunk; a.gate_f32 = gate_dtype == VT_F32;
-    a.scale = scale; a.cap = cap; a.dist_r1 = dist_r1; a.dist_r2 = dist_r2; a.score_shift = score_shift;
+    a.max_blocks = max_blocks; a.num_pages = num_pages; a.window = window; a.chunk = chunk; a.keep_first = keep_first;
+    a.gate_f32 = gate_dtype == VT_F32; a.scale = scale; a.cap = cap; a.dist_r1 = dist_r1; a.dist_r2 = dist_r2; a.score_shift = score_shift;
     a.sigmoid_weights = sigmoid_weights; a.gate_wide = gate_wide;
     attn_masked_decode_kernel<<<dim3(splits, G * HT, n), 256, 0, stream>>>(a);
     VT_CHECK_LAUNCH("vt_attn_masked_decode");
@@ -746,7 +770,7 @@ extern "C" int vt_attn_masked_mfma_dims(int* key_dim, int* value_dim) {
 extern "C" int vt_attn_masked_mfma(const void* q, const void* k_pages, const void* v_pages, const int* positions,
                                    const int* tok_entry, const int* block_table, const int* tiles, int n_tiles,
                                    const void* gate, int gate_dtype, long long ldg, void* out, int H, int G, int D, int Dv,
-                                   int page_size, int max_blocks, int num_pages, int window, int chunk, float scale,
+                                   int page_size, int max_blocks, int num_pages, int window, int chunk, int keep_first, float scale,
                                    float cap, const float* sink, const float* slopes, const float* dist_r1,
                                    const float* dist_r2, const float* score_shift, int sigmoid_weights, int gate_wide,
                                    hipStream_t stream) {
@@ -759,13 +783,15 @@ extern "C" int vt_attn_masked_mfma(const void* q, const void* k_pages, const voi
     VT_REQUIRE(page_size > 0 && page_size % 16 == 0 && max_blocks > 0 && num_pages > 0,
                "vt_attn_masked_mfma: pages of %d keys (a multiple of 16)", page_size);
     VT_REQUIRE(window >= 0 && chunk >= 0 && cap >= 0.f, "vt_attn_masked_mfma: bad mask or cap");
+    VT_REQUIRE(keep_first >= 0 && (keep_first == 0 || (window > 0 && chunk == 0)),
+               "vt_attn_masked_mfma: %d first keys kept beside window %d, chunk %d", keep_first, window, chunk);
     VT_REQUIRE(!gate || gate_dtype == VT_F32 || gate_dtype == VT_BF16, "vt_attn_masked_mfma: gate dtype %d", gate_dtype);
     if (n_tiles == 0) return 0;
     MfmaArgs a;
     a.q = (const bf16_t*)q; a.k_pages = (const bf16_t*)k_pages; a.v_pages = (const bf16_t*)v_pages; a.positions = positions;
     a.tok_entry = tok_entry; a.block_table = block_table; a.tiles = tiles; a.gate = gate; a.out = (bf16_t*)out; a.ldg = ldg;
     a.n_tiles = n_tiles; a.H = H; a.G = G; a.page_size = page_size; a.max_blocks = max_blocks; a.num_pages = num_pages;
-    a.window = window; a.chunk = chunk; a.gate_f32 = gate_dtype == VT_F32; a.scale = scale; a.cap = cap;
+    a.window = window; a.chunk = chunk; a.keep_first = keep_first; a.gate_f32 = gate_dtype == VT_F32; a.scale = scale; a.cap = cap;
     a.sink = sink; a.slopes = slopes; a.dist_r1 = dist_r1; a.dist_r2 = dist_r2; a.score_shift = score_shift;
     a.sigmoid_weights = sigmoid_weights; a.gate_wide = gate_wide;
     const long long items = (long long)n_tiles * H;

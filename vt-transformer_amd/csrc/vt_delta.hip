@@ -370,18 +370,21 @@ extern "C" int vt_delta_rule(const void* qkv, int dtype, const void* ba, int ba_
 // ---------------------------------------------------------------------------
 // out[t][h][:] = o[t][h][:] / sqrt(mean(o^2) + eps) * w[h * w_stride + :] * act(gate[t][h][:]); gate[t * ldg + h * Dv + j];
 // act: silu (gate_kind 0) or sigmoid (1); w_stride 0: one weight vector for all heads, Dv: one per head
-template <typename TG, typename TO>
-__global__ __launch_bounds__(64) void gated_rmsnorm_kernel(const float* __restrict__ o, const float* __restrict__ w,
+// A wave per (token, head); wide heads (a norm over all heads of a token at once is one such head) take a block of four.
+template <typename TG, typename TO, int THREADS>
+__global__ __launch_bounds__(THREADS) void gated_rmsnorm_kernel(const float* __restrict__ o, const float* __restrict__ w,
                                                            const TG* __restrict__ gate, long long ldg, TO* __restrict__ out,
                                                            int H, int Dv, float eps, int w_stride, int gate_kind) {
+    __shared__ float red[16];
     const int t = blockIdx.x, h = blockIdx.y, lane = threadIdx.x;
     const float* row = o + ((size_t)t * H + h) * Dv;
     const float* wh = w + (size_t)h * w_stride;
     float ss = 0.f;
-    for (int j = lane; j < Dv; j += 64) ss = fmaf(row[j], row[j], ss);
-    ss = wave_sum(ss);
+    for (int j = lane; j < Dv; j += THREADS) ss = fmaf(row[j], row[j], ss);
+    if constexpr (THREADS > 64) ss = block_sum(ss, red);
+    else ss = wave_sum(ss);
     const float rinv = 1.0f / sqrtf(ss / (float)Dv + eps);
-    for (int j = lane; j < Dv; j += 64) {
+    for (int j = lane; j < Dv; j += THREADS) {
         const float z = load_f32<TG>(gate, (size_t)t * ldg + (size_t)h * Dv + j);
         const float g = gate_kind ? 1.0f / (1.0f + expf(-z)) : silu_f(z);
         store_f32<TO>(out, ((size_t)t * H + h) * Dv + j, row[j] * rinv * wh[j] * g);
@@ -397,13 +400,14 @@ extern "C" int vt_gated_rmsnorm(const float* o, const float* w, const void* gate
     if (n == 0) return 0;
     const dim3 grid(n, H);
     const int ws = w_per_head ? Dv : 0;
-    if (gate_dtype == VT_F32 && out_dtype == VT_F32)
-        gated_rmsnorm_kernel<float, float><<<grid, 64, 0, stream>>>(o, w, (const float*)gate, ldg, (float*)out, H, Dv, eps, ws, gate_kind);
-    else if (gate_dtype == VT_F32 && out_dtype == VT_BF16)
-        gated_rmsnorm_kernel<float, bf16_t><<<grid, 64, 0, stream>>>(o, w, (const float*)gate, ldg, (bf16_t*)out, H, Dv, eps, ws, gate_kind);
-    else if (gate_dtype == VT_BF16 && out_dtype == VT_BF16)
-        gated_rmsnorm_kernel<bf16_t, bf16_t><<<grid, 64, 0, stream>>>(o, w, (const bf16_t*)gate, ldg, (bf16_t*)out, H, Dv, eps, ws, gate_kind);
+#define VT_GNORM(TG, TO) do { \
+        if (Dv > 512) gated_rmsnorm_kernel<TG, TO, 256><<<grid, 256, 0, stream>>>(o, w, (const TG*)gate, ldg, (TO*)out, H, Dv, eps, ws, gate_kind); \
+        else gated_rmsnorm_kernel<TG, TO, 64><<<grid, 64, 0, stream>>>(o, w, (const TG*)gate, ldg, (TO*)out, H, Dv, eps, ws, gate_kind); } while (0)
+    if (gate_dtype == VT_F32 && out_dtype == VT_F32) VT_GNORM(float, float);
+    else if (gate_dtype == VT_F32 && out_dtype == VT_BF16) VT_GNORM(float, bf16_t);
+    else if (gate_dtype == VT_BF16 && out_dtype == VT_BF16) VT_GNORM(bf16_t, bf16_t);
     else return vt_fail("vt_gated_rmsnorm: dtypes %d -> %d are not handled", gate_dtype, out_dtype);
+#undef VT_GNORM
     VT_CHECK_LAUNCH("vt_gated_rmsnorm");
     return 0;
 }

@@ -667,6 +667,36 @@ extern "C" int vt_gated_act(const void* gu, int in_dtype, void* out, int out_dty
     return 0;
 }
 
+// out <- max(x, 0)^2, element by element (in and out may be one tensor)
+template <typename TI, typename TO>
+__global__ __launch_bounds__(256) void squared_relu_kernel(const TI* x, TO* out, long long n4, long long n) {
+    const long long i = (long long)blockIdx.x * 256 + threadIdx.x;
+    if (i < n4) {
+        float4 v = load4(x + 4 * i);
+        v.x = fmaxf(v.x, 0.f); v.y = fmaxf(v.y, 0.f); v.z = fmaxf(v.z, 0.f); v.w = fmaxf(v.w, 0.f);
+        store4(out + 4 * i, make_float4(v.x * v.x, v.y * v.y, v.z * v.z, v.w * v.w));
+    } else {
+        const long long j = 4 * n4 + (i - n4);
+        if (j < n) {
+            const float v = fmaxf(load_f32<TI>(x, (size_t)j), 0.f);
+            store_f32<TO>(out, (size_t)j, v * v);
+        }
+    }
+}
+extern "C" int vt_squared_relu(const void* x, int in_dtype, void* out, int out_dtype, long long n, hipStream_t stream) {
+    VT_REQUIRE(n >= 0, "vt_squared_relu: bad size");
+    if (n == 0) return 0;
+    const long long n4 = (((uintptr_t)x | (uintptr_t)out) & 15) ? 0 : n / 4;
+    const long long blocks = (n4 + (n - 4 * n4) + 255) / 256;
+    VT_REQUIRE(blocks <= 0x7fffffff, "vt_squared_relu: too many elements");
+    if (in_dtype == VT_F32 && out_dtype == VT_F32) squared_relu_kernel<float, float><<<(unsigned)blocks, 256, 0, stream>>>((const float*)x, (float*)out, n4, n);
+    else if (in_dtype == VT_F32 && out_dtype == VT_BF16) squared_relu_kernel<float, bf16_t><<<(unsigned)blocks, 256, 0, stream>>>((const float*)x, (bf16_t*)out, n4, n);
+    else if (in_dtype == VT_BF16 && out_dtype == VT_BF16) squared_relu_kernel<bf16_t, bf16_t><<<(unsigned)blocks, 256, 0, stream>>>((const bf16_t*)x, (bf16_t*)out, n4, n);
+    else return vt_fail("vt_squared_relu: unknown dtypes %d -> %d", in_dtype, out_dtype);
+    VT_CHECK_LAUNCH("vt_squared_relu");
+    return 0;
+}
+
 // x <- cap * tanh(x / cap), in place (logits bounded to (-cap, cap))
 __global__ void tanh_cap_kernel(float* __restrict__ x, long long n, float cap) {
     for (long long i = (long long)blockIdx.x * blockDim.x + threadIdx.x; i < n; i += (long long)gridDim.x * blockDim.x)

@@ -163,7 +163,17 @@ struct NormLink {
     int n_ssq;
     float eps;
     GateForm gate;             // (rides along: the gate's form of a gated product)
+    int act;                   // (likewise: what a plain product's result passes, behind the bias: ACT_*)
 };
+#define ACT_NONE 0
+#define ACT_SQUARED_RELU 1
+__device__ __forceinline__ float plain_act(float v, int act) {
+    if (act == ACT_SQUARED_RELU) {
+        v = fmaxf(v, 0.f);
+        v *= v;
+    }
+    return v;
+}
 #define SSQ_STRIDE(N) ((N) <= 16 ? 16 : 64)
 
 // Consumer of a NormLink at 17 to 64 rows (shares 64 floats apart): 1/sqrt(sum / K + eps) of every row into
@@ -469,7 +479,10 @@ __global__ __launch_bounds__(WPB * 64) void gemm_skinny_kernel(const void* __res
                     u += bias[Mout + m];
                 }
                 v = gate_form(v, u, link.gate);
-            } else if (bias) v += bias[m];
+            } else {
+                if (bias) v += bias[m];
+                v = plain_act(v, link.act);
+            }
             if (resid) v += resid[(size_t)n * Mout + m];
             store_f32<TO>(y, (size_t)n * Mout + m, v);
             if (link.xn_out) {
@@ -669,8 +682,9 @@ __global__ __launch_bounds__((WM + 1) * 64) void gemm_mid_kernel(const bf16_t* _
                         u += bias[Mout + m];
                     }
                     v = gate_form(v, u, link.gate);
-                } else if (bias && blockIdx.z == 0) {
-                    v += bias[m];
+                } else {
+                    if (bias && blockIdx.z == 0) v += bias[m];
+                    if (!split) v = plain_act(v, link.act);
                 }
                 if (split) partial[((size_t)blockIdx.z * N + n) * Mout + m] = v;
                 else store_f32<TO>(y, (size_t)n * Mout + m, v);
@@ -788,6 +802,7 @@ __global__ __launch_bounds__(WPB * 64) __attribute__((amdgpu_waves_per_eu(2, 4))
             if (m < Mout && n < N) {
                 if (consumes) v *= link_rinv[n];
                 if (bias) v += bias[m];
+                v = plain_act(v, link.act);
                 if (resid) v += resid[(size_t)n * Mout + m];
                 store_f32<TO>(y, (size_t)n * Mout + m, v);
                 if (link.xn_out) {
@@ -827,9 +842,10 @@ static int launch_rows(const bf16_t* x, const bf16_t* wp, const float* bias, TO*
     return 0;
 }
 
-// y[i] = sum over splits of partial[s][i], added in split order
+// y[i] = act(sum over splits of partial[s][i]), added in split order
 template <typename TO>
-__global__ void sum_partials_kernel(const float* __restrict__ partial, TO* __restrict__ y, size_t n, int splits) {
+__global__ void sum_partials_kernel(const float* __restrict__ partial, TO* __restrict__ y, size_t n, int splits,
+                                    int act) {
     const size_t i = ((size_t)blockIdx.x * blockDim.x + threadIdx.x) * 4;
     if (i >= n) return;
     if (i + 4 <= n) {
@@ -838,12 +854,13 @@ __global__ void sum_partials_kernel(const float* __restrict__ partial, TO* __res
             float4 b = *(const float4*)(partial + (size_t)s * n + i);
             a.x += b.x; a.y += b.y; a.z += b.z; a.w += b.w;
         }
-        store_f32<TO>(y, i, a.x); store_f32<TO>(y, i + 1, a.y); store_f32<TO>(y, i + 2, a.z); store_f32<TO>(y, i + 3, a.w);
+        store_f32<TO>(y, i, plain_act(a.x, act)); store_f32<TO>(y, i + 1, plain_act(a.y, act));
+        store_f32<TO>(y, i + 2, plain_act(a.z, act)); store_f32<TO>(y, i + 3, plain_act(a.w, act));
     } else {
         for (size_t j = i; j < n; ++j) {
             float a = partial[j];
             for (int s = 1; s < splits; ++s) a += partial[(size_t)s * n + j];
-            store_f32<TO>(y, j, a);
+            store_f32<TO>(y, j, plain_act(a, act));
         }
     }
 }
@@ -895,7 +912,7 @@ __device__ __forceinline__ float packed_at(const bf16_t* wp, int KT, int m, int 
 template <bool SWIGLU, typename TO>
 __global__ void gemm_plain_kernel(const bf16_t* __restrict__ x, const bf16_t* __restrict__ wp,
                                   const float* __restrict__ bias, TO* __restrict__ y, int N, int Mout, int K, int KT,
-                                  int up_tiles, GateForm gate) {
+                                  int up_tiles, GateForm gate, int act) {
     int m = blockIdx.x * blockDim.x + threadIdx.x, n = blockIdx.y;
     if (m >= Mout) return;
     const bf16_t* xr = x + (size_t)n * K;
@@ -908,8 +925,9 @@ __global__ void gemm_plain_kernel(const bf16_t* __restrict__ x, const bf16_t* __
             u += bias[Mout + m];
         }
         v = gate_form(v, u, gate);
-    } else if (bias) {
-        v += bias[m];
+    } else {
+        if (bias) v += bias[m];
+        v = plain_act(v, act);
     }
     store_f32<TO>(y, (size_t)n * Mout + m, v);
 }
@@ -999,7 +1017,7 @@ extern "C" long long vt_linear_bf16_workspace(int N, int M, int K, int gated) {
 
 // gain != null: x is the fp32 residual stream and the RMSNorm (gain, eps) is part of the product (up to 16 tokens);
 // resid != null: the result is added to it (up to 64 tokens).
-static const NormLink NO_LINK = {nullptr, nullptr, nullptr, nullptr, 0, 0.f, {1.f, 0.f, 0.f, 0.f}};
+static const NormLink NO_LINK = {nullptr, nullptr, nullptr, nullptr, 0, 0.f, {1.f, 0.f, 0.f, 0.f}, ACT_NONE};
 
 // shares of the rows' sums of squares that a producing product of this shape writes (0: it cannot produce)
 extern "C" int vt_linear_bf16_link_shares(int N, int M, int K) {
@@ -1033,7 +1051,7 @@ static int linear_bf16(const void* xv, const bf16_t* wp, const float* bias, TO* 
     VT_REQUIRE((((uintptr_t)wp) & 15) == 0, "vt_linear_bf16: the packed matrix is not 16-byte aligned");
     if (K % 8 != 0 || ((uintptr_t)x & 15)) {
         VT_REQUIRE(N <= 65535, "vt_linear_bf16: too many rows (%d) for the any-shape kernel", N);
-        gemm_plain_kernel<SWIGLU, TO><<<dim3((Mout + 255) / 256, N), 256, 0, stream>>>(x, wp, bias, y, N, Mout, K, KT, up_tiles, link.gate);
+        gemm_plain_kernel<SWIGLU, TO><<<dim3((Mout + 255) / 256, N), 256, 0, stream>>>(x, wp, bias, y, N, Mout, K, KT, up_tiles, link.gate, link.act);
         VT_CHECK_LAUNCH("vt_linear_bf16(plain)");
         return 0;
     }
@@ -1064,7 +1082,7 @@ static int linear_bf16(const void* xv, const bf16_t* wp, const float* bias, TO* 
         VT_REQUIRE(!link.ssq_in || grid.y == 1, "vt_linear_bf16: a prepared norm is taken with up to 64 rows (N=%d)", N);
         // the product takes the norm in front (link.ssq_in); the one behind is prepared where the sums are added up
         NormLink in = NO_LINK;
-        in.ssq_in = link.ssq_in; in.n_ssq = link.n_ssq; in.eps = link.eps; in.gate = link.gate;
+        in.ssq_in = link.ssq_in; in.n_ssq = link.n_ssq; in.eps = link.eps; in.gate = link.gate; in.act = link.act;
 #define VT_MID__(W, O, T) do { \
             static bool lds_set = false; \
             if (!lds_set) { \
@@ -1097,7 +1115,7 @@ static int linear_bf16(const void* xv, const bf16_t* wp, const float* bias, TO* 
                     return 0;
                 }
             }
-            sum_partials_kernel<TO><<<(unsigned)((n / 4 + 255) / 256 + 1), 256, 0, stream>>>(workspace, y, n, splits);
+            sum_partials_kernel<TO><<<(unsigned)((n / 4 + 255) / 256 + 1), 256, 0, stream>>>(workspace, y, n, splits, link.act);
             VT_CHECK_LAUNCH("vt_linear_bf16(sum)");
         }
         return 0;
@@ -1131,6 +1149,18 @@ extern "C" int vt_linear_bf16(const void* x, const void* wp, const float* bias, 
     if (out_dtype == VT_F32) return linear_bf16<false, float>(x, (const bf16_t*)wp, bias, (float*)y, workspace, N, M, K, nullptr, 0.f, nullptr, stream);
     if (out_dtype == VT_BF16) return linear_bf16<false, bf16_t>(x, (const bf16_t*)wp, bias, (bf16_t*)y, workspace, N, M, K, nullptr, 0.f, nullptr, stream);
     return vt_fail("vt_linear_bf16: unknown out dtype %d", out_dtype);
+}
+
+// y[N, M] = act(x[N, K] . W[M, K]^T + bias), act one of ACT_*: the activation on the float32 sums
+extern "C" int vt_linear_bf16_act(const void* x, const void* wp, const float* bias, void* y, int out_dtype, float* workspace,
+                                  int N, int M, int K, int act, hipStream_t stream) {
+    VT_REQUIRE(N >= 0 && M > 0 && K > 0, "vt_linear_bf16_act: bad sizes N=%d M=%d K=%d", N, M, K);
+    VT_REQUIRE(act == ACT_NONE || act == ACT_SQUARED_RELU, "vt_linear_bf16_act: unknown activation %d", act);
+    NormLink link = NO_LINK;
+    link.act = act;
+    if (out_dtype == VT_F32) return linear_bf16<false, float>(x, (const bf16_t*)wp, bias, (float*)y, workspace, N, M, K, nullptr, 0.f, nullptr, stream, link);
+    if (out_dtype == VT_BF16) return linear_bf16<false, bf16_t>(x, (const bf16_t*)wp, bias, (bf16_t*)y, workspace, N, M, K, nullptr, 0.f, nullptr, stream, link);
+    return vt_fail("vt_linear_bf16_act: unknown out dtype %d", out_dtype);
 }
 
 // ---------------------------------------------------------------------------
@@ -1199,7 +1229,7 @@ extern "C" int vt_linear_bf16_link(const void* x, const void* wp, const float* b
                                    void* xn_out, const float* gain_next, float* ssq_out, hipStream_t stream) {
     VT_REQUIRE(N >= 0 && M > 0 && K > 0, "vt_linear_bf16_link: bad sizes N=%d M=%d K=%d", N, M, K);
     VT_REQUIRE(ssq_in || xn_out, "vt_linear_bf16_link: neither end of a norm: use vt_linear_bf16");
-    const NormLink link = {(bf16_t*)xn_out, gain_next, ssq_out, ssq_in, n_ssq, eps_in, {1.f, 0.f, 0.f, 0.f}};
+    const NormLink link = {(bf16_t*)xn_out, gain_next, ssq_out, ssq_in, n_ssq, eps_in, {1.f, 0.f, 0.f, 0.f}, ACT_NONE};
     return linear_bf16<false, float>(x, (const bf16_t*)wp, bias, y, workspace, N, M, K, nullptr, 0.f, resid, stream, link);
 }
 
@@ -1208,7 +1238,7 @@ extern "C" int vt_gated_linear_bf16_link(const void* x, const void* wp, void* y,
                                          const float* ssq_in, int n_ssq, float eps_in, hipStream_t stream) {
     VT_REQUIRE(N >= 0 && I > 0 && K > 0, "vt_gated_linear_bf16_link: bad sizes N=%d I=%d K=%d", N, I, K);
     VT_REQUIRE(ssq_in, "vt_gated_linear_bf16_link: no sums of squares: use vt_gated_linear_bf16");
-    const NormLink link = {nullptr, nullptr, nullptr, ssq_in, n_ssq, eps_in, {1.f, 0.f, 0.f, 0.f}};
+    const NormLink link = {nullptr, nullptr, nullptr, ssq_in, n_ssq, eps_in, {1.f, 0.f, 0.f, 0.f}, ACT_NONE};
     if (out_dtype == VT_F32) return linear_bf16<true, float>(x, (const bf16_t*)wp, nullptr, (float*)y, nullptr, N, I, K, nullptr, 0.f, nullptr, stream, link);
     if (out_dtype == VT_BF16) return linear_bf16<true, bf16_t>(x, (const bf16_t*)wp, nullptr, (bf16_t*)y, nullptr, N, I, K, nullptr, 0.f, nullptr, stream, link);
     return vt_fail("vt_gated_linear_bf16_link: unknown out dtype %d", out_dtype);
@@ -1224,7 +1254,7 @@ extern "C" int vt_gated_linear_bf16_form(const void* x, const void* wp, const fl
     VT_REQUIRE(N >= 0 && I > 0 && K > 0, "vt_gated_linear_bf16_form: bad sizes N=%d I=%d K=%d", N, I, K);
     VT_REQUIRE(!(gain && ssq_in), "vt_gated_linear_bf16_form: a norm in front is applied here or was prepared, not both");
     VT_REQUIRE(alpha > 0.f && limit >= 0.f, "vt_gated_linear_bf16_form: bad gate (alpha %g, limit %g)", alpha, limit);
-    const NormLink link = {nullptr, nullptr, nullptr, ssq_in, ssq_in ? n_ssq : 0, ssq_in ? eps : 0.f, {alpha, limit, shift, cubic}};
+    const NormLink link = {nullptr, nullptr, nullptr, ssq_in, ssq_in ? n_ssq : 0, ssq_in ? eps : 0.f, {alpha, limit, shift, cubic}, ACT_NONE};
     const float* g = ssq_in ? nullptr : gain;
     if (out_dtype == VT_F32) return linear_bf16<true, float>(x, (const bf16_t*)wp, bias, (float*)y, nullptr, N, I, K, g, eps, nullptr, stream, link);
     if (out_dtype == VT_BF16) return linear_bf16<true, bf16_t>(x, (const bf16_t*)wp, bias, (bf16_t*)y, nullptr, N, I, K, g, eps, nullptr, stream, link);

@@ -11,7 +11,8 @@
 //                    in_scale (the choice's score where the score multiplies the expert's input, else 1), rounded to the
 //                    runtime's type as an expert's input is; f(g) = g sigmoid(alpha g (1 + cubic g^2)).
 //   vt_moe_down:     out[t] = sum over the token's choices, in their order, of out_scale * W_down,e act.
-// These two read an expert's matrices once per token that chose it: the arrangement for few tokens, where every chosen
+//   vt_moe_up:       the first half of experts without a gate: act = max(W_up,e xe, 0)^2 for every (token, choice).
+// These three read an expert's matrices once per token that chose it: the arrangement for few tokens, where every chosen
 // expert's matrices have to be read anyway.  (Many tokens go through vt_moe_sort and the grouped products below.)
 // A pair whose id is negative has no expert: no product is made for it and nothing of it is written or read.
 // Every sum is taken in an order that depends on the sizes alone, so a token's result does not depend on its batch.
@@ -251,6 +252,27 @@ __global__ __launch_bounds__(256) void moe_gate_up_kernel(const TI* __restrict__
     }
 }
 
+// w_up: [E][F][W]; act: [pairs][F] = max(W_up,e x, 0)^2
+template <typename TI, typename TW>
+__global__ __launch_bounds__(256) void moe_up_kernel(const TI* __restrict__ x, const TW* __restrict__ w_up, const int* __restrict__ ids,
+                                                     TI* __restrict__ act, int W, int F, int top) {
+    extern __shared__ float xs[];       // W
+    const int p = blockIdx.x;
+    const int e = ids[p];
+    if (e < 0) return;
+    for (int j = threadIdx.x; j < W; j += 256) xs[j] = load_f32<TI>(x, (size_t)(p / top) * W + j);
+    __syncthreads();
+    const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
+    const TW* we = w_up + (size_t)e * F * W;
+#pragma unroll
+    for (int i = 0; i < MOE_OUTS_PER_WAVE; ++i) {
+        const int f = blockIdx.y * MOE_OUTS_PER_BLOCK + wave * MOE_OUTS_PER_WAVE + i;
+        if (f >= F) break;
+        const float u = fmaxf(wave_dot<TW>(we + (size_t)f * W, xs, W, lane), 0.f);
+        if (lane == 0) store_f32<TI>(act, (size_t)p * F + f, u * u);
+    }
+}
+
 // w_down: [E][W][F]; out [n][W] float32
 template <typename TI, typename TW>
 __global__ __launch_bounds__(256) void moe_down_kernel(const TI* __restrict__ act, const TW* __restrict__ w_down,
@@ -301,6 +323,22 @@ extern "C" int vt_moe_gate_up(const void* x, int dtype, const void* w_gu, int w_
         moe_gate_up_kernel<bf16_t, bf16_t><<<grid, 256, lds, stream>>>((const bf16_t*)x, (const bf16_t*)w_gu, ids, wts, (bf16_t*)act, W, F, top, scale_input, alpha, cubic);
     else return vt_fail("vt_moe_gate_up: dtypes %d / %d are not handled", dtype, w_dtype);
     VT_CHECK_LAUNCH("vt_moe_gate_up");
+    return 0;
+}
+
+extern "C" int vt_moe_up(const void* x, int dtype, const void* w_up, int w_dtype, const int* ids, void* act, int n, int E, int W,
+                         int F, int top, hipStream_t stream) {
+    VT_REQUIRE(n >= 0 && E > 0 && W > 0 && F > 0 && top > 0, "vt_moe_up: bad sizes");
+    VT_REQUIRE(W <= 16384 && (F + MOE_OUTS_PER_BLOCK - 1) / MOE_OUTS_PER_BLOCK <= 65535, "vt_moe_up: width %d or experts' size %d is too large", W, F);
+    if (n == 0) return 0;
+    const dim3 grid(n * top, (F + MOE_OUTS_PER_BLOCK - 1) / MOE_OUTS_PER_BLOCK);
+    const size_t lds = (size_t)W * sizeof(float);
+    if (dtype == VT_F32 && w_dtype == VT_F32)
+        moe_up_kernel<float, float><<<grid, 256, lds, stream>>>((const float*)x, (const float*)w_up, ids, (float*)act, W, F, top);
+    else if (dtype == VT_BF16 && w_dtype == VT_BF16)
+        moe_up_kernel<bf16_t, bf16_t><<<grid, 256, lds, stream>>>((const bf16_t*)x, (const bf16_t*)w_up, ids, (bf16_t*)act, W, F, top);
+    else return vt_fail("vt_moe_up: dtypes %d / %d are not handled", dtype, w_dtype);
+    VT_CHECK_LAUNCH("vt_moe_up");
     return 0;
 }
 
@@ -402,12 +440,18 @@ extern "C" int vt_moe_sort(const int* ids, int* plan, int pairs, int E, hipStrea
     return 0;
 }
 
+// What a grouped product is: the second one of an expert (from the activations, float32 results), or the first one of
+// gated experts (gate and up rows together) or of experts without a gate (activation: max(., 0)^2).
+#define GR_DOWN 0
+#define GR_GATED 1
+#define GR_UP 2
+
 struct GroupedArgs {
-    const bf16_t* x;        // gated: the tokens [n][K]; else the activations in sorted order [P][K]
+    const bf16_t* x;        // gated, up: the tokens [n][K]; down: the activations in sorted order [P][K]
     const bf16_t* w;        // gated: [E][2 M][K] (gate rows, then up rows); else [E][M][K]
     const int* plan;
     const float* wts;       // the pairs' scores
-    void* out;              // gated: activations in sorted order [P][M], 16 bits; else float32 [P][M] in the pairs' order
+    void* out;              // gated, up: activations in sorted order [P][M], 16 bits; down: float32 [P][M] in the pairs' order
     int P, K, M, top, T, scale;
     float alpha, cubic;
 };
@@ -418,10 +462,21 @@ union MoeFrag {
     vt_lowp8_t v;
 };
 
+__device__ __forceinline__ uint2 moe_squared_relu4(const moe_f32x4_t& v) {
+    float u[4];
+#pragma unroll
+    for (int q = 0; q < 4; ++q) {
+        u[q] = fmaxf(v[q], 0.f);
+        u[q] *= u[q];
+    }
+    return make_uint2(vt_pack2(u[0], u[1]), vt_pack2(u[2], u[3]));
+}
+
 __device__ __forceinline__ unsigned moe_scale2(unsigned u, float s) { return vt_pack2(lowp_lo(u) * s, lowp_hi(u) * s); }
 
-template <bool GATED>
+template <int MODE>
 __global__ __launch_bounds__(256) void moe_grouped_kernel(GroupedArgs a) {
+    constexpr bool GATED = MODE == GR_GATED, TOKENS = MODE != GR_DOWN;
     const int tile = blockIdx.y;
     if (tile >= a.plan[0]) return;
     const int* order = a.plan + 1;
@@ -442,15 +497,18 @@ __global__ __launch_bounds__(256) void moe_grouped_kernel(GroupedArgs a) {
     for (int i = 0; i < 4; ++i) {
         const int row = lr + 32 * i;
         const int rr = min(row, rows - 1);          // beyond the tile's pairs the last one again (never stored)
-        if (GATED) {
+        if (TOKENS) {
             const int p = order[row0 + rr];
             xrow[i] = a.x + (size_t)(p / a.top) * K;
             xscale[i] = scaled ? a.wts[p] : 1.f;
-            const int f = min((int)blockIdx.x * 64 + (row & 63), M - 1);
-            wrow[i] = a.w + ((size_t)e * 2 * M + (row < 64 ? f : M + f)) * K;
         } else {
             xrow[i] = a.x + (size_t)(row0 + rr) * K;
             xscale[i] = 1.f;
+        }
+        if (GATED) {
+            const int f = min((int)blockIdx.x * 64 + (row & 63), M - 1);
+            wrow[i] = a.w + ((size_t)e * 2 * M + (row < 64 ? f : M + f)) * K;
+        } else {
             wrow[i] = a.w + ((size_t)e * M + min((int)blockIdx.x * GR_FB + row, M - 1)) * K;
         }
     }
@@ -544,6 +602,19 @@ __global__ __launch_bounds__(256) void moe_grouped_kernel(GroupedArgs a) {
                 *(uint2*)(act + (size_t)(row0 + row) * M + f) = o;
             }
         }
+    } else if (TOKENS) {
+        bf16_t* act = (bf16_t*)a.out;
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+            const int row = 64 * wt + 16 * i + r;
+            if (row >= rows) continue;
+#pragma unroll
+            for (int j = 0; j < 4; ++j) {
+                const int m = (int)blockIdx.x * GR_FB + 64 * wf + 16 * j + 4 * g;
+                if (m >= M) continue;
+                *(uint2*)(act + (size_t)(row0 + row) * M + m) = moe_squared_relu4(acc[j][i]);
+            }
+        }
     } else {
         float* out = (float*)a.out;
 #pragma unroll
@@ -572,8 +643,9 @@ __global__ __launch_bounds__(256) void moe_grouped_kernel(GroupedArgs a) {
 // and up to 16 pairs at a time; its four waves split K in turns of 64 (a cache line of every row) and read their
 // operands straight from memory (a lane 16 bytes of its row), two turns' loads in flight; the waves' sums meet in LDS in a fixed order.  Sixteen
 // rows to a block give eight times the blocks of the tiled kernel, which is what fills the GPU when the pairs are few.
-template <bool GATED>
+template <int MODE>
 __global__ __launch_bounds__(256) void moe_few_kernel(GroupedArgs a) {
+    constexpr bool GATED = MODE == GR_GATED, TOKENS = MODE != GR_DOWN;
     const int tile = blockIdx.y;
     if (tile >= a.plan[0]) return;
     const int* order = a.plan + 1;
@@ -593,7 +665,7 @@ __global__ __launch_bounds__(256) void moe_few_kernel(GroupedArgs a) {
         const int pr = row0 + min(sub + r, rows - 1);       // beyond the tile's pairs the last one again (never stored)
         const bf16_t* xrow;
         float xs = 1.f;
-        if (GATED) {
+        if (TOKENS) {
             const int p = order[pr];
             xrow = a.x + (size_t)(p / a.top) * K;
             if (scaled) xs = a.wts[p];
@@ -654,6 +726,8 @@ __global__ __launch_bounds__(256) void moe_few_kernel(GroupedArgs a) {
                     o.x = vt_pack2(v4[0], v4[1]);
                     o.y = vt_pack2(v4[2], v4[3]);
                     *(uint2*)((bf16_t*)a.out + (size_t)(row0 + row) * M + m) = o;
+                } else if (TOKENS) {
+                    *(uint2*)((bf16_t*)a.out + (size_t)(row0 + row) * M + m) = moe_squared_relu4(acc0);
                 } else {
                     const int p = order[row0 + row];
                     const float s = a.scale ? a.wts[p] : 1.f;
@@ -684,9 +758,10 @@ __global__ __launch_bounds__(256) void moe_combine_kernel(const float* __restric
 static int grouped_ready() {
     static int done = 0;
     if (done) return 0;
-    hipError_t e1 = hipFuncSetAttribute((const void*)moe_grouped_kernel<true>, hipFuncAttributeMaxDynamicSharedMemorySize, GR_LDS_BYTES);
-    hipError_t e2 = hipFuncSetAttribute((const void*)moe_grouped_kernel<false>, hipFuncAttributeMaxDynamicSharedMemorySize, GR_LDS_BYTES);
-    if (e1 != hipSuccess || e2 != hipSuccess) return vt_fail("vt_moe: the grouped products' LDS could not be set");
+    hipError_t e1 = hipFuncSetAttribute((const void*)moe_grouped_kernel<GR_GATED>, hipFuncAttributeMaxDynamicSharedMemorySize, GR_LDS_BYTES);
+    hipError_t e2 = hipFuncSetAttribute((const void*)moe_grouped_kernel<GR_DOWN>, hipFuncAttributeMaxDynamicSharedMemorySize, GR_LDS_BYTES);
+    hipError_t e3 = hipFuncSetAttribute((const void*)moe_grouped_kernel<GR_UP>, hipFuncAttributeMaxDynamicSharedMemorySize, GR_LDS_BYTES);
+    if (e1 != hipSuccess || e2 != hipSuccess || e3 != hipSuccess) return vt_fail("vt_moe: the grouped products' LDS could not be set");
     done = 1;
     return 0;
 }
@@ -704,9 +779,26 @@ extern "C" int vt_moe_gate_up_grouped(const void* x, const void* w_gu, const int
     const int P = n * top, T = vt_moe_plan_tiles(P, E);
     VT_REQUIRE(T <= 65535, "vt_moe_gate_up_grouped: too many pairs (%d)", P);
     GroupedArgs a = {(const bf16_t*)x, (const bf16_t*)w_gu, plan, wts, act, P, W, F, top, T, scale_input, alpha, cubic};
-    if (P <= GR_FEW_PAIRS) moe_few_kernel<true><<<dim3((F + 15) / 16, T), 256, 0, stream>>>(a);
-    else moe_grouped_kernel<true><<<dim3((F + 63) / 64, T), 256, GR_LDS_BYTES, stream>>>(a);
+    if (P <= GR_FEW_PAIRS) moe_few_kernel<GR_GATED><<<dim3((F + 15) / 16, T), 256, 0, stream>>>(a);
+    else moe_grouped_kernel<GR_GATED><<<dim3((F + 63) / 64, T), 256, GR_LDS_BYTES, stream>>>(a);
     VT_CHECK_LAUNCH("vt_moe_gate_up_grouped");
+    return 0;
+}
+
+// the same for experts without a gate: act = max(W_up,e x, 0)^2; w_up [E][F][W]
+extern "C" int vt_moe_up_grouped(const void* x, const void* w_up, const int* plan, void* act, int n, int E, int W, int F, int top,
+                                 hipStream_t stream) {
+    VT_REQUIRE(n >= 0 && E > 0 && E <= GR_MAX_EXPERTS && top > 0, "vt_moe_up_grouped: bad sizes");
+    VT_REQUIRE(W > 0 && F > 0 && W % 8 == 0 && F % 8 == 0, "vt_moe_up_grouped: width %d and experts' size %d (multiples of 8)", W, F);
+    VT_REQUIRE(!(((uintptr_t)x | (uintptr_t)w_up | (uintptr_t)act) & 15), "vt_moe_up_grouped: operands must be 16-byte aligned");
+    if (n == 0) return 0;
+    if (grouped_ready()) return -1;
+    const int P = n * top, T = vt_moe_plan_tiles(P, E);
+    VT_REQUIRE(T <= 65535, "vt_moe_up_grouped: too many pairs (%d)", P);
+    GroupedArgs a = {(const bf16_t*)x, (const bf16_t*)w_up, plan, nullptr, act, P, W, F, top, T, 0, 1.f, 0.f};
+    if (P <= GR_FEW_PAIRS) moe_few_kernel<GR_UP><<<dim3((F + 15) / 16, T), 256, 0, stream>>>(a);
+    else moe_grouped_kernel<GR_UP><<<dim3((F + GR_FB - 1) / GR_FB, T), 256, GR_LDS_BYTES, stream>>>(a);
+    VT_CHECK_LAUNCH("vt_moe_up_grouped");
     return 0;
 }
 
@@ -725,8 +817,8 @@ extern "C" int vt_moe_down_grouped(const void* act, const void* w_down, const in
     VT_REQUIRE(T <= 65535, "vt_moe_down_grouped: too many pairs (%d)", P);
     GroupedArgs a = {(const bf16_t*)act, (const bf16_t*)w_down, plan, wts, top == 1 && out ? (void*)out : (void*)y, P, F, W, top, T,
                      scale_output, 1.f, 0.f};
-    if (P <= GR_FEW_PAIRS) moe_few_kernel<false><<<dim3((W + 15) / 16, T), 256, 0, stream>>>(a);
-    else moe_grouped_kernel<false><<<dim3((W + GR_FB - 1) / GR_FB, T), 256, GR_LDS_BYTES, stream>>>(a);
+    if (P <= GR_FEW_PAIRS) moe_few_kernel<GR_DOWN><<<dim3((W + 15) / 16, T), 256, 0, stream>>>(a);
+    else moe_grouped_kernel<GR_DOWN><<<dim3((W + GR_FB - 1) / GR_FB, T), 256, GR_LDS_BYTES, stream>>>(a);
     VT_CHECK_LAUNCH("vt_moe_down_grouped");
     if (top > 1 && out) {
         const long long total4 = (long long)n * (W / 4);

@@ -248,6 +248,17 @@ def gated_act(gu: torch.Tensor, out: torch.Tensor, alpha: float = 1.0, limit: fl
     return out
 
 
+def squared_relu(x: torch.Tensor, out: torch.Tensor) -> torch.Tensor:
+    """out = max(x, 0)^2, element by element; out may be x."""
+    _chk(x, "squared_relu.x")
+    _chk(out, "squared_relu.out", None, x.shape)
+    if out.dtype == torch.float32 and x.dtype != torch.float32:
+        raise KernelError("squared_relu: float32 results need float32 inputs")
+    _run(load_lib("vt_elementwise", half=_half(x, out)), "vt_squared_relu", _ptr(x), _i(_code(x)), _ptr(out), _i(_code(out)),
+         ctypes.c_longlong(x.numel()), _stream())
+    return out
+
+
 def tanh_cap(x: torch.Tensor, cap: float) -> torch.Tensor:
     """x <- cap * tanh(x / cap), in place; float32."""
     _chk(x, "tanh_cap.x", torch.float32)
@@ -395,6 +406,7 @@ def linear_bf16_workspace(n: int, m: int, k: int) -> int:
 
 NORM_MAX_ROWS = 16         # rows up to which the few-row product applies an RMSNorm in front
 LINK_MAX_ROWS = 64         # rows up to which a product takes a norm that the product in front has prepared
+PLAIN_ACTS = {"squared_relu": 1}    # activations that a plain product can put on its sums
 _adds_residual = {}
 
 
@@ -410,14 +422,14 @@ def linear_bf16_adds_residual(n: int, m: int, k: int) -> bool:
 
 def linear_bf16(x: torch.Tensor, w, bias: Optional[torch.Tensor], out: torch.Tensor,
                 workspace: Optional[torch.Tensor] = None, norm_gain: Optional[torch.Tensor] = None,
-                norm_eps: float = 0.0, residual: Optional[torch.Tensor] = None) -> torch.Tensor:
+                norm_eps: float = 0.0, residual: Optional[torch.Tensor] = None, act: Optional[str] = None) -> torch.Tensor:
     """Few rows (decoding, short portions): W is read once per 64 rows.  w: a PackedMatrix (a plain [m, k] tensor
     is packed on the spot, which costs more than the product).  Shapes whose k range is split over blocks need
     `workspace` (float32, at least linear_bf16_workspace(n, m, k) elements).
     float32 output: with norm_gain (up to 16 rows), x is the float32 residual stream and rmsnorm(x; gain, eps) is
     what gets multiplied; with residual (where linear_bf16_adds_residual says so; float32 [n, m], may be `out`), out =
     residual + the product (17 to 64 rows of a shape whose k range is split: by the launch that adds the partial sums,
-    which needs the workspace)."""
+    which needs the workspace).  act (with neither of these): one of PLAIN_ACTS on the float32 sums."""
     n, k = x.shape
     lp = _lowp((w.data if isinstance(w, PackedMatrix) else w), "linear_bf16.w")
     if not isinstance(w, PackedMatrix):
@@ -427,6 +439,8 @@ def linear_bf16(x: torch.Tensor, w, bias: Optional[torch.Tensor], out: torch.Ten
     if w.cols != k or w.halves != 1:
         raise KernelError(f"linear_bf16: x [{n}, {k}] does not fit a packed matrix [{w.rows}, {w.cols}] x {w.halves}")
     fused = norm_gain is not None or residual is not None
+    if act is not None and (fused or act not in PLAIN_ACTS):
+        raise KernelError(f"linear_bf16: activation {act!r} ({', '.join(PLAIN_ACTS)}; without norm and residual)")
     _chk(x, "linear_bf16.x", torch.float32 if norm_gain is not None else lp)
     _chk(w.data, "linear_bf16.w", lp)
     _chk(out, "linear_bf16.out", torch.float32 if fused else None, (n, m))
@@ -457,6 +471,10 @@ def linear_bf16(x: torch.Tensor, w, bias: Optional[torch.Tensor], out: torch.Ten
         _chk(workspace, "linear_bf16.workspace", torch.float32)
         if workspace.numel() < need:
             raise KernelError(f"linear_bf16: workspace of {workspace.numel()} floats, need {need}")
+    if act is not None:
+        _run(load_lib("vt_gemm_bf16", half=_half(w.data, x, out)), "vt_linear_bf16_act", _ptr(x), _ptr(w.data), _ptr(bias), _ptr(out),
+             _i(_code(out)), _ptr(workspace if need else None), _i(n), _i(m), _i(k), _i(PLAIN_ACTS[act]), _stream())
+        return out
     _run(load_lib("vt_gemm_bf16", half=_half(w.data, x, out)), "vt_linear_bf16", _ptr(x), _ptr(w.data), _ptr(bias), _ptr(out), _i(_code(out)),
          _ptr(workspace if need else None), _i(n), _i(m), _i(k), _stream())
     return out
@@ -907,10 +925,11 @@ def attention_masked(q: torch.Tensor, k_pages: torch.Tensor, v_pages: torch.Tens
                      gate: Optional[torch.Tensor] = None, gate_column: int = 0, sink: Optional[torch.Tensor] = None,
                      slopes: Optional[torch.Tensor] = None, dist_log: Optional[tuple] = None,
                      score_shift: Optional[torch.Tensor] = None, sigmoid_weights: bool = False,
-                     gate_wide: bool = False) -> torch.Tensor:
+                     gate_wide: bool = False, keep_first: int = 0) -> torch.Tensor:
     """out [n, H * Dv] = softmax over the seen keys of cap * tanh(scale q.k / cap) (cap 0: scale q.k), times V, times
     sigmoid(gate[:, gate_column + head]) if `gate` (a 2-d tensor whose rows are the tokens') is given.  Key j is seen
-    from position i if j <= i, i - j < window (0: unbounded) and j is in i's chunk of `chunk` positions (0: unbounded).
+    from position i if j <= i, i - j < window (0: unbounded) and j is in i's chunk of `chunk` positions (0: unbounded);
+    keep_first (with a window and no chunks): the keys j < keep_first are seen from every later position as well.
     slopes (float32 [H]): slopes[h] * (i - j) is taken off the score; sink (float32 [H]): exp(sink[h]) is added to the
     softmax's denominator.  dist_log (r1, r2), float32 [H] each: r1[h] ln(1 + r2[h] (i - j)) is taken off the score;
     score_shift (float32 [H]): a number per head added to every score; sigmoid_weights: the weight of a seen key is
@@ -944,7 +963,7 @@ def attention_masked(q: torch.Tensor, k_pages: torch.Tensor, v_pages: torch.Tens
     _run(load_lib("vt_attn_masked", half=_half(q, gate)), "vt_attn_masked", _ptr(q), _ptr(k_pages), _ptr(v_pages), _i(_code(q)),
          _ptr(positions), _ptr(tok_entry), _ptr(block_table), gptr, _i(gcode), ctypes.c_longlong(ldg), _ptr(out), _i(n),
          _i(n_heads), _i(n_kv), _i(key_dim), _i(value_dim), _i(page_size), _i(block_table.shape[1]), _i(num_pages),
-         _i(window), _i(chunk), _f(scale), _f(cap), _ptr(sink), _ptr(slopes), _ptr(r1), _ptr(r2), _ptr(score_shift),
+         _i(window), _i(chunk), _i(keep_first), _f(scale), _f(cap), _ptr(sink), _ptr(slopes), _ptr(r1), _ptr(r2), _ptr(score_shift),
          _i(1 if sigmoid_weights else 0), _i(1 if (gate_wide and gate is not None) else 0), _stream())
     return out
 
@@ -982,7 +1001,7 @@ def attention_masked_mfma(q: torch.Tensor, k_pages: torch.Tensor, v_pages: torch
                           gate_column: int = 0, sink: Optional[torch.Tensor] = None,
                           slopes: Optional[torch.Tensor] = None, dist_log: Optional[tuple] = None,
                           score_shift: Optional[torch.Tensor] = None, sigmoid_weights: bool = False,
-                          gate_wide: bool = False) -> torch.Tensor:
+                          gate_wide: bool = False, keep_first: int = 0) -> torch.Tensor:
     """attention_masked for the 16-bit types on the matrix cores.  tiles: int32 [n_tiles, 2], (first row, rows) of
     runs of up to 16 consecutive tokens of one request that together cover every token of the step once."""
     n = q.shape[0]
@@ -1015,21 +1034,21 @@ def attention_masked_mfma(q: torch.Tensor, k_pages: torch.Tensor, v_pages: torch
     _run(load_lib("vt_attn_masked_mfma", (key_dim, value_dim), half=_half(q, gate)), "vt_attn_masked_mfma", _ptr(q), _ptr(k_pages),
          _ptr(v_pages), _ptr(positions), _ptr(tok_entry), _ptr(block_table), _ptr(tiles), _i(tiles.numel() // 2), gptr,
          _i(gcode), ctypes.c_longlong(ldg), _ptr(out), _i(n_heads), _i(n_kv), _i(key_dim), _i(value_dim), _i(page_size),
-         _i(block_table.shape[1]), _i(num_pages), _i(window), _i(chunk), _f(scale), _f(cap), _ptr(sink), _ptr(slopes),
+         _i(block_table.shape[1]), _i(num_pages), _i(window), _i(chunk), _i(keep_first), _f(scale), _f(cap), _ptr(sink), _ptr(slopes),
          _ptr(r1), _ptr(r2), _ptr(score_shift), _i(1 if sigmoid_weights else 0),
          _i(1 if (gate_wide and gate is not None) else 0), _stream())
     return out
 
 
-def attention_masked_decode_splits(n: int, n_heads: int, n_kv: int, max_len: int, reach: int = 0) -> int:
+def attention_masked_decode_splits(n: int, n_heads: int, n_kv: int, max_len: int, reach: int = 0, keep_first: int = 0) -> int:
     """Into how many blocks of four waves a decoding step's keys are dealt per (token, group of heads): enough to give
     every compute unit a few waves, no more than there are turns of 32 keys in the longest sequence, or in the `reach`
-    positions that a mask leaves of it (0: all).  It depends on the number of tokens, the mask and the engine's limits
+    positions that a mask leaves of it (0: all) and its first `keep_first`.  It depends on the number of tokens, the mask and the engine's limits
     alone, so that a recorded step can be replayed."""
     tiles = max(1, n) * n_kv * (-(-(n_heads // n_kv) // 16))
     most = max(1, max_len // 128)
     if reach > 0:
-        turns = (reach + 14) // 32 + 1          # (the first turn starts at a multiple of 16)
+        turns = (reach + 14) // 32 + 1 + -(-keep_first // 32)       # (the first turn starts at a multiple of 16)
         most = min(most, -(-turns // 4))
     return int(max(1, min(-(-512 // tiles), most, 16)))
 
@@ -1041,7 +1060,7 @@ def attention_masked_decode(q: torch.Tensor, k_pages: torch.Tensor, v_pages: tor
                             gate_column: int = 0, sink: Optional[torch.Tensor] = None,
                             slopes: Optional[torch.Tensor] = None, dist_log: Optional[tuple] = None,
                             score_shift: Optional[torch.Tensor] = None, sigmoid_weights: bool = False,
-                            gate_wide: bool = False) -> torch.Tensor:
+                            gate_wide: bool = False, keep_first: int = 0) -> torch.Tensor:
     """attention_masked for steps of single tokens in the 16-bit types on the matrix cores: the rows of a product are
     the query heads that share a key/value head.  part: float32 scratch of attention_masked_decode_scratch floats."""
     n = q.shape[0]
@@ -1073,7 +1092,7 @@ def attention_masked_decode(q: torch.Tensor, k_pages: torch.Tensor, v_pages: tor
          _ptr(k_pages), _ptr(v_pages), _ptr(positions), _ptr(tok_entry), _ptr(block_table), gptr, _i(gcode),
          ctypes.c_longlong(ldg), _ptr(out), _ptr(part), ctypes.c_longlong(part.numel()), _i(splits), _i(n), _i(n_heads),
          _i(n_kv), _i(key_dim), _i(value_dim), _i(page_size), _i(block_table.shape[1]), _i(num_pages), _i(window), _i(chunk),
-         _f(scale), _f(cap), _ptr(sink), _ptr(slopes), _ptr(r1), _ptr(r2), _ptr(score_shift), _i(1 if sigmoid_weights else 0),
+         _i(keep_first), _f(scale), _f(cap), _ptr(sink), _ptr(slopes), _ptr(r1), _ptr(r2), _ptr(score_shift), _i(1 if sigmoid_weights else 0),
          _i(1 if (gate_wide and gate is not None) else 0), _stream())
     return out
 
@@ -1406,6 +1425,37 @@ def matrix_memory(x: torch.Tensor, q_column: int, k_column: int, v_column: int, 
 
 
 # ---------------------------------------------------------------------------
+# linear attention with a constant decay per head (vt_linear_attn.hip)
+def decayed_attention(x: torch.Tensor, q_column: int, k_column: int, v_column: int, decay: torch.Tensor, state: torch.Tensor,
+                      entry_start: torch.Tensor, slots: torch.Tensor, out: torch.Tensor, n_heads: int, key_dim: int,
+                      value_dim: int, silu: bool = True, single: bool = False) -> torch.Tensor:
+    """S <- decay[h] S + k v^T, o = S^T q per head over the tokens of every entry, from and into state[slot] ([H, Dv, D]
+    float32).  x: a 2-d tensor whose rows are the tokens', with H heads of D queries from q_column, of D keys from
+    k_column and of Dv values from v_column; silu: all three pass a SiLU first (in float32).  single: every entry brings
+    exactly one token.  decay [H] float32; out [n, H * Dv] float32."""
+    n = x.shape[0]
+    hd = n_heads * key_dim
+    _chk(x, "decayed_attention.x")
+    if x.dim() != 2 or min(q_column, k_column, v_column) < 0 or \
+            x.shape[1] < max(max(q_column, k_column) + hd, v_column + n_heads * value_dim):
+        raise KernelError(f"decayed_attention.x: shape {tuple(x.shape)} does not hold its columns")
+    _chk(decay, "decayed_attention.decay", torch.float32, (n_heads,))
+    _chk(out, "decayed_attention.out", torch.float32, (n, n_heads * value_dim))
+    _chk(entry_start, "decayed_attention.entry_start", torch.int32)
+    _chk(slots, "decayed_attention.slots", torch.int32)
+    if not 1 <= key_dim <= DELTA_MAX_KEY_DIM:
+        raise KernelError(f"decayed_attention: keys of {key_dim} (up to {DELTA_MAX_KEY_DIM})")
+    entries = entry_start.numel() - 1
+    if single and entries != n:
+        raise KernelError(f"decayed_attention: {n} tokens are not one for each of {entries} entries")
+    sp, ss = _state_rows(state, "decayed_attention", n_heads * key_dim * value_dim)
+    _run(load_lib("vt_linear_attn", half=_half(x)), "vt_decayed_attn", _ptr(x), _i(_code(x)), ctypes.c_longlong(x.stride(0)),
+         _i(q_column), _i(k_column), _i(v_column), _ptr(decay), sp, ss, _ptr(entry_start), _ptr(slots), _ptr(out), _i(entries),
+         _i(n_heads), _i(key_dim), _i(value_dim), _i(1 if silu else 0), _i(1 if single else 0), _stream())
+    return out
+
+
+# ---------------------------------------------------------------------------
 # several residual streams and the token shift (vt_streams.hip)
 STREAMS_MAX = 8
 
@@ -1527,6 +1577,37 @@ def moe_gate_up(x: torch.Tensor, w_gu: torch.Tensor, ids: torch.Tensor, weights:
     return act
 
 
+def moe_up(x: torch.Tensor, w_up: torch.Tensor, ids: torch.Tensor, act: torch.Tensor) -> torch.Tensor:
+    """act[t * top + k] = max(W_up,e x[t], 0)^2 for e = ids[t, k] (a pair whose id is negative is left out): the first half
+    of experts without a gate; w_up [E, F, W]; act [n * top, F] in x's type."""
+    n, w = x.shape
+    e, f, _ = w_up.shape
+    top = ids.shape[1]
+    _chk(x, "moe_up.x")
+    _chk(w_up, "moe_up.w_up", x.dtype, (e, f, w))
+    _chk(ids, "moe_up.ids", torch.int32, (n, top))
+    _chk(act, "moe_up.act", x.dtype, (n * top, f))
+    _run(load_lib("vt_moe", half=_half(x)), "vt_moe_up", _ptr(x), _i(_code(x)), _ptr(w_up), _i(_code(w_up)), _ptr(ids), _ptr(act),
+         _i(n), _i(e), _i(w), _i(f), _i(top), _stream())
+    return act
+
+
+def moe_up_grouped(x: torch.Tensor, w_up: torch.Tensor, plan: torch.Tensor, act: torch.Tensor, top: int) -> torch.Tensor:
+    """moe_up on the matrix cores: act [n * top, F] in the plan's order (pairs sorted by expert).  x [n, W] and w_up
+    [E, F, W] of one 16-bit type."""
+    n, w = x.shape
+    e, f, _ = w_up.shape
+    _chk(x, "moe_up_grouped.x")
+    if x.dtype not in LOWP:
+        raise KernelError("moe_up_grouped: a 16-bit type is needed")
+    _chk(w_up, "moe_up_grouped.w_up", x.dtype, (e, f, w))
+    _chk(plan, "moe_up_grouped.plan", torch.int32, (moe_plan_size(n * top, e),))
+    _chk(act, "moe_up_grouped.act", x.dtype, (n * top, f))
+    _run(load_lib("vt_moe", half=_half(x)), "vt_moe_up_grouped", _ptr(x), _ptr(w_up), _ptr(plan), _ptr(act), _i(n), _i(e), _i(w),
+         _i(f), _i(top), _stream())
+    return act
+
+
 def moe_down(act: torch.Tensor, w_down: torch.Tensor, ids: torch.Tensor, weights: torch.Tensor, out: torch.Tensor,
              scale_output: bool) -> torch.Tensor:
     """out[t] = sum_k (weights[t, k] if scale_output) * W_down,e act[t * top + k], e = ids[t, k], in the order of k
@@ -1614,7 +1695,7 @@ def moe_down_grouped(act: torch.Tensor, w_down: torch.Tensor, plan: torch.Tensor
 
 # ---------------------------------------------------------------------------
 # a sublayer's result, whole or in pieces, and the norm on it (vt_output_norm.hip)
-def _pieces(who: str, n: int, w: int, y, choices, ids, id_weights, x):
+def _pieces(who: str, n: int, w: int, y, choices, ids, id_weights, x, pair=None):
     """Checks of the pieces of a sublayer's result; returns the arguments that describe them."""
     top = 0
     if choices is not None:
@@ -1629,41 +1710,63 @@ def _pieces(who: str, n: int, w: int, y, choices, ids, id_weights, x):
         _chk(x, who + ".x", None, (n, w))
     if y is not None:
         _chk(y, who + ".y", None, (n, w))
+    y2 = gain1 = gain2 = None
+    scale1 = scale2 = pair_eps = 0.0
+    if pair is not None:
+        if y is not None:
+            raise KernelError(who + ": a pair of results stands in y's place")
+        (y, gain1, scale1), (y2, gain2, scale2), pair_eps = pair
+        for t, g, name in ((y, gain1, "pair[0]"), (y2, gain2, "pair[1]")):
+            _chk(t, f"{who}.{name}", None, (n, w))
+            _chk(g, f"{who}.{name}.gain", torch.float32, (w,))
     if choices is None and id_weights is None and y is None:
         raise KernelError(who + ": no pieces")
     return (_ptr(choices), _ptr(ids if choices is not None else None), _i(top), _ptr(id_weights),
             _ptr(x if id_weights is not None else None), _i(_code(x) if id_weights is not None else F32), _ptr(y),
-            _i(_code(y) if y is not None else F32))
+            _i(_code(y) if y is not None else F32), _ptr(y2), _i(_code(y2) if y2 is not None else F32), _ptr(gain1), _ptr(gain2),
+            _f(scale1), _f(scale2), _f(pair_eps))
+
+
+def _pair_tensors(pair):
+    return (pair[0][0], pair[1][0]) if pair is not None else ()
 
 
 def sublayer_sum(out: torch.Tensor, y: Optional[torch.Tensor] = None, choices: Optional[torch.Tensor] = None,
                  ids: Optional[torch.Tensor] = None, id_weights: Optional[torch.Tensor] = None,
-                 x: Optional[torch.Tensor] = None) -> torch.Tensor:
+                 x: Optional[torch.Tensor] = None, pair: Optional[tuple] = None) -> torch.Tensor:
     """out[t] = sum_k choices[t * top + k] + id_weights[t] * x[t] + y[t], every kind of piece optional: choices float32
     [n * top, W], of which those with a negative id (ids int32 [n, top]; None: all count) are left out; x and y [n, W]
-    float32 or 16-bit; out [n, W] float32."""
+    float32 or 16-bit; out [n, W] float32.  pair ((y1, gain1, scale1), (y2, gain2, scale2), eps), in y's place: the sum of
+    scale * gain * y / sqrt(mean(y^2) + eps) over both (gains float32 [W])."""
     n, w = out.shape
     _chk(out, "sublayer_sum.out", torch.float32)
-    args = _pieces("sublayer_sum", n, w, y, choices, ids, id_weights, x)
-    _run(load_lib("vt_output_norm", half=_half(x if id_weights is not None else None, y)), "vt_sublayer_sum", _ptr(out), *args, _i(n),
-         _i(w), _stream())
+    args = _pieces("sublayer_sum", n, w, y, choices, ids, id_weights, x, pair)
+    _run(load_lib("vt_output_norm", half=_half(x if id_weights is not None else None, y, *_pair_tensors(pair))), "vt_sublayer_sum",
+         _ptr(out), *args, _i(n), _i(w), _stream())
     return out
 
 
 def output_norm_add(h: torch.Tensor, gain: torch.Tensor, eps: float, mult: float, y: Optional[torch.Tensor] = None,
                     choices: Optional[torch.Tensor] = None, ids: Optional[torch.Tensor] = None,
                     id_weights: Optional[torch.Tensor] = None, x: Optional[torch.Tensor] = None,
-                    copy: Optional[torch.Tensor] = None) -> torch.Tensor:
+                    copy: Optional[torch.Tensor] = None, pair: Optional[tuple] = None,
+                    next_gain: Optional[torch.Tensor] = None, next_eps: float = 0.0) -> torch.Tensor:
     """h[t] += mult * gain * u[t] / sqrt(mean(u[t]^2) + eps) with u what `sublayer_sum` gives for the same pieces (x may
-    be h itself); h float32 [n, W], changed in place.  copy [n, W]: the new h in this tensor's type as well."""
+    be h itself); h float32 [n, W], changed in place.  copy [n, W]: the new h in this tensor's type as well, or with
+    next_gain (float32 [W]) next_gain * h / sqrt(mean(h^2) + next_eps) in its place."""
     n, w = h.shape
     _chk(h, "output_norm_add.h", torch.float32)
     _chk(gain, "output_norm_add.gain", torch.float32, (w,))
     if copy is not None:
         _chk(copy, "output_norm_add.copy", None, (n, w))
-    args = _pieces("output_norm_add", n, w, y, choices, ids, id_weights, x)
-    _run(load_lib("vt_output_norm", half=_half(x if id_weights is not None else None, y, copy)), "vt_output_norm_add", _ptr(h), *args,
-         _ptr(gain), _ptr(copy), _i(_code(copy) if copy is not None else F32), _i(n), _i(w), _f(mult), _f(eps), _stream())
+    if next_gain is not None:
+        _chk(next_gain, "output_norm_add.next_gain", torch.float32, (w,))
+        if copy is None:
+            raise KernelError("output_norm_add: a norm behind without a tensor for it")
+    args = _pieces("output_norm_add", n, w, y, choices, ids, id_weights, x, pair)
+    _run(load_lib("vt_output_norm", half=_half(x if id_weights is not None else None, y, copy, *_pair_tensors(pair))),
+         "vt_output_norm_add", _ptr(h), *args, _ptr(gain), _ptr(copy), _i(_code(copy) if copy is not None else F32), _ptr(next_gain),
+         _f(next_eps), _i(n), _i(w), _f(mult), _f(eps), _stream())
     return h
 
 

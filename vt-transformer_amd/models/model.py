@@ -15,8 +15,8 @@ import torch
 from ..config.base import LayerSpec, ModelSpec, PartSpec
 from ..kernels import ops
 from ..parts.linear import linear
-from ..parts.base import (BLOCKS, EMBEDDINGS, FEED_FORWARDS, HEADS, MIXERS, NORMS, NormedInput, Part, Registry,
-                          Runtime, StreamCopy, TensorDecl)
+from ..parts.base import (BLOCKS, EMBEDDINGS, FEED_FORWARDS, HEADS, MIXERS, NORMS, NormedInput, NormedStream, Part,
+                          Registry, Runtime, StreamCopy, TensorDecl)
 
 
 def settle(h: torch.Tensor, delta):
@@ -124,6 +124,8 @@ class DecoderModel:
             block = self.layers[entry.layer]
             if isinstance(delta, StreamCopy) and not getattr(block, "takes_stream_copy", False):
                 delta = None                # (nothing is left to be added; this block goes on from the stream)
+            if isinstance(delta, NormedStream) and not getattr(block, "takes_normed_stream", False):
+                delta = None
             if isinstance(delta, tuple) and (entry.inject or entry.offset_row is not None
                                              or not getattr(block, "takes_pair", False)):
                 h, delta = settle(h, delta), None
@@ -152,7 +154,7 @@ class DecoderModel:
                 h, delta = block.forward(h, delta, ctx, caches[i], states[i])
         if ctx.n_logit_rows == 0:
             return None
-        if isinstance(delta, (NormedInput, StreamCopy)):
+        if isinstance(delta, (NormedInput, NormedStream, StreamCopy)):
             delta = None
         if isinstance(delta, tuple):
             if getattr(self.final_norm, "takes_pair", False) and not self.streams:

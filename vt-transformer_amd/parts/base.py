@@ -10,14 +10,15 @@ Interfaces (N = tokens of the step, H = model width):
 
   Norm            forward(h[N,H] fp32, delta[N,H] or None, rows=None) -> normed [N or R, H] in the runtime's dtype.
                   With `delta`, h += delta happens first (and is stored in h unless `rows` picks rows).
-                  Optional: forward_output(h, y, mult, copy), the norm on a sublayer's output: h += mult * norm(y), with
-                  y a tensor or SublayerPieces, and the new h in `copy` as well.
+                  Optional: forward_output(h, y, mult, copy, behind), the norm on a sublayer's output: h += mult * norm(y),
+                  with y a tensor or SublayerPieces, and the new h (or the norm `behind` of it) in `copy` as well.
   PositionEncoding
                   rotary_tables(n_positions) -> (cos, sin) fp32 [n_positions, dims/2] or None if the
                   encoding is not a rotation that the fused kernel can apply;
                   apply(q, k, positions) -> (q, k) otherwise.
   Mixer           forward(x[N,H], ctx, cache, state) -> [N,H]; cache_need() / state_need() say what the cache
                   manager has to hold for it (keys and values in pages; fixed-size state per request).
+                  One that `hands_pieces` takes pieces=True and may then return its result not added up (SublayerPieces).
                   Optional: prepare_step(ctx) -> {key: int32 array} or None, called on the host once per step
                   before the step's metadata goes to the device; what it returns is found in ctx.extra[key] on
                   the device when the part runs (work items of its kernels, lengths they read from memory).
@@ -30,7 +31,7 @@ Interfaces (N = tokens of the step, H = model width):
   Block           forward(h, delta, ctx, cache, state) -> (h, delta): arranges two norms, a mixer and a
                   feed-forward around the fp32 residual stream h.  `delta` is a layer output that has
                   not been added to h yet, so that the next norm can fuse the addition (or None, or what a
-                  block of its kind can use: NormedInput, a pair of tensors, StreamCopy).
+                  block of its kind can use: NormedInput, a pair of tensors, StreamCopy, NormedStream).
 
 The reference's counterpart is the set of `op.*` words that a model program
 strings together (v1/tensortype/nn_operators.cpp:530-576) and its user words
@@ -100,9 +101,10 @@ class CacheNeed:
     tensors: Tuple[PageTensor, ...]
     window: int = 0  # 0: every token stays; W: a token is dead once W later tokens exist
     page_multiple: int = 1  # the mixer's kernels take pages whose size is a multiple of this many tokens
+    keep_first: int = 0  # with a window: a sequence's first so many tokens stay all the same
 
     def group_key(self):
-        return (self.tensors, self.window)
+        return (self.tensors, self.window, self.keep_first)
 
     def same_layout(self, other: "CacheNeed") -> bool:
         """Whether a mixer with this need can read pages that a mixer with the other need writes."""
@@ -235,20 +237,30 @@ class StreamCopy:
         self.x = x
 
 
+class NormedStream:
+    """What a block whose sublayers' outputs are normed hands on where the block behind starts with a norm: nothing is left
+    to be added to the stream, and `x` is that norm (`norm`) of it, as the norm on the last sublayer's output has written
+    it.  Whoever does not read it goes on from the stream."""
+
+    def __init__(self, x: torch.Tensor, norm):
+        self.x, self.norm = x, norm
+
+
 class SublayerPieces:
     """A sublayer's result that has not been added up: rows of a mixture's choices [tokens * top, width] (those with a
-    negative id left out), a weight per token on the sublayer's own input, and a result that every token has, each
+    negative id left out), a weight per token on the sublayer's own input, and a result that every token has (or, in
+    its place, a pair ((y1, gain1, scale1), (y2, gain2, scale2), eps) of results that are normed, scaled and added), each
     optional.  A norm on the output takes the pieces as they are (`RMSNorm.forward_output`); `materialize()` is their
     sum as a tensor, for whoever cannot."""
 
     def __init__(self, rt: "Runtime", rows: int, width: int, y: Optional[torch.Tensor] = None,
                  choices: Optional[torch.Tensor] = None, ids: Optional[torch.Tensor] = None,
-                 id_weights: Optional[torch.Tensor] = None, x: Optional[torch.Tensor] = None):
+                 id_weights: Optional[torch.Tensor] = None, x: Optional[torch.Tensor] = None, pair: Optional[tuple] = None):
         self.rt, self.rows, self.width = rt, int(rows), int(width)
-        self.y, self.choices, self.ids, self.id_weights, self.x = y, choices, ids, id_weights, x
+        self.y, self.choices, self.ids, self.id_weights, self.x, self.pair = y, choices, ids, id_weights, x, pair
 
-    def as_args(self) -> Dict[str, Optional[torch.Tensor]]:
-        return dict(y=self.y, choices=self.choices, ids=self.ids, id_weights=self.id_weights, x=self.x)
+    def as_args(self) -> Dict[str, object]:
+        return dict(y=self.y, choices=self.choices, ids=self.ids, id_weights=self.id_weights, x=self.x, pair=self.pair)
 
     def materialize(self) -> torch.Tensor:
         from ..kernels import ops

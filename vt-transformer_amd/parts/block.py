@@ -22,7 +22,7 @@ from typing import Callable, Dict, Optional, Tuple
 import torch
 
 from ..kernels import ops
-from .base import BLOCKS, NormedInput, Part, Runtime, StateNeed, StreamCopy, TensorDecl
+from .base import BLOCKS, NormedInput, NormedStream, Part, Runtime, StateNeed, StreamCopy, TensorDecl
 from .linear import can_fuse, linear
 
 
@@ -31,6 +31,7 @@ class PreNormBlock(Part):
     norm_roles = ("input", "post_mixer")
     replayable = True
     takes_next_norm = True      # forward(..., next_norm=): the norm that the layer behind this one starts with
+    takes_normed_stream = True  # forward(h, delta, ...) with delta a NormedStream
 
     def __init__(self, *, rt: Runtime, norms, mixer, feed_forward, prefix: str = "", width: int = 0):
         self.rt = rt
@@ -66,6 +67,8 @@ class PreNormBlock(Part):
         takes = getattr(part, "takes_normed_input", False)
         if isinstance(delta, NormedInput):
             x = delta if (delta.norm is norm and takes) else norm.forward(h, None)
+        elif isinstance(delta, NormedStream):
+            x = delta.x if delta.norm is norm else norm.forward(h, None)
         elif fuse and delta is None and getattr(norm, "rms_fusable", False) and takes:
             x = NormedInput(h, norm)
         else:
@@ -181,6 +184,69 @@ class OutputNormBlock(Part):
             more = {"pieces": True} if getattr(self.feed_forward, "hands_pieces", False) else {}
             self.norm_ff.forward_output(h, self.feed_forward.forward(x, ctx, **more), self.mult, copy)
         return h, StreamCopy(x)
+
+
+@BLOCKS.register("sandwich")
+class SandwichNormBlock(Part):
+    """A norm in front of each sublayer and another one on its result:
+
+        x <- x + norm_1b(mixer(norm_1(x)));   x <- x + norm_2b(feed_forward(norm_2(x)))
+
+    The norm on a result, the addition to the stream and the norm in front of the sublayer behind it are one kernel
+    (`forward_output` with `behind`), which also adds up a result that is handed on in pieces; the last one of a layer
+    makes the norm that the layer behind starts with, where that layer can take it (NormedStream)."""
+
+    norm_roles = ("input", "mixer_output", "post_mixer", "feed_forward_output")
+    replayable = True
+    takes_next_norm = True
+    takes_normed_stream = True
+
+    def __init__(self, *, rt: Runtime, norms, mixer, feed_forward, prefix: str = "", width: int = 0, idle_norms=()):
+        """idle_norms: the second sublayer's norms' tensors of a layer without a feed-forward, which a checkpoint may hold and
+        which are not read."""
+        self.rt, self.width = rt, int(width)
+        self.norm_in, self.norm_mixer = norms["input"], norms["mixer_output"]
+        self.mixer = mixer
+        self.feed_forward = feed_forward
+        self.norm_post = norms["post_mixer"] if feed_forward is not None else None
+        self.norm_ff = norms["feed_forward_output"] if feed_forward is not None else None
+        self.idle_norms = tuple(prefix + n for n in idle_norms) if feed_forward is None else ()
+
+    def parts(self):
+        if self.feed_forward is None:
+            return [self, self.norm_in, self.mixer, self.norm_mixer]
+        return [self, self.norm_in, self.mixer, self.norm_mixer, self.norm_post, self.feed_forward, self.norm_ff]
+
+    @property
+    def first_norm(self):
+        return self.norm_in
+
+    def tensors(self) -> Dict[str, TensorDecl]:
+        return {n: TensorDecl((self.width,), "gain", optional=True) for n in self.idle_norms}
+
+    def _join(self, h, norm, y, behind):
+        """h += norm(y); returns the norm `behind` of the new h (None: nobody asks for it)."""
+        if behind is None:
+            norm.forward_output(h, y)
+            return None
+        x = self.rt.buffer("sandwich.normed", tuple(h.shape), self.rt.dtype)
+        norm.forward_output(h, y, copy=x, behind=behind)
+        return x
+
+    def forward(self, h: torch.Tensor, delta, ctx, cache, state, next_norm=None) -> Tuple[torch.Tensor, object]:
+        if isinstance(delta, NormedStream):
+            x = delta.x if delta.norm is self.norm_in else self.norm_in.forward(h, None)
+        else:
+            x = self.norm_in.forward(h, delta if isinstance(delta, torch.Tensor) else None)
+        if not getattr(next_norm, "rms_fusable", False):
+            next_norm = None
+        pieces = {"pieces": True} if getattr(self.mixer, "hands_pieces", False) else {}
+        y = self.mixer.forward(x, ctx, cache, state, **pieces)
+        x = self._join(h, self.norm_mixer, y, self.norm_post if self.feed_forward is not None else next_norm)
+        if self.feed_forward is not None:
+            pieces = {"pieces": True} if getattr(self.feed_forward, "hands_pieces", False) else {}
+            x = self._join(h, self.norm_ff, self.feed_forward.forward(x, ctx, **pieces), next_norm)
+        return h, (NormedStream(x, next_norm) if x is not None else None)
 
 
 @BLOCKS.register("hyper")

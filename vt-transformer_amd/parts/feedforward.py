@@ -1,4 +1,4 @@
-"""Gated feed-forward: down( act(gate(x)) * up(x) ).
+"""Feed-forwards: gated, down( act(gate(x)) * up(x) ), and without a gate, down( act(up(x)) ).
 
 The reference's order (v1/models/qwen2-7b/inference_fp16.dag:333-337): up
 projection (mlp.w2), gate projection (mlp.w1), silu(gate) * up
@@ -155,3 +155,38 @@ class GatedMLP(Part):
             gu = linear(rt, x, self.w_gu, None, "mlp.gu", packed=self.p_gu if self.w_gu is None else None)
             ops.silu_mul(gu, act)
         return linear(rt, act, self.w_down, None, "mlp.down", packed=self.p_down, residual=residual, hand_on=hand_on)
+
+
+@FEED_FORWARDS.register("plain_mlp")
+class PlainMLP(Part):
+    """The feed-forward without a gate: down( act(up(x)) ), act the square of ReLU.  With few tokens the activation is
+    applied to the float32 accumulators inside the first product's kernel."""
+
+    replayable = True
+
+    def __init__(self, *, rt: Runtime, width: int, prefix: str, intermediate_size: int, activation: str = "squared_relu",
+                 names: Optional[Dict[str, str]] = None, weight_suffix: str = ""):
+        """names: the two matrices' names behind the prefix; weight_suffix: what follows them in the tensors' names."""
+        if activation not in ops.PLAIN_ACTS:
+            raise ValueError(f"activation '{activation}' is not supported ({', '.join(ops.PLAIN_ACTS)})")
+        self.rt, self.width, self.inter, self.act = rt, int(width), int(intermediate_size), activation
+        if self.inter <= 0:
+            raise ValueError(f"a feed-forward of {self.inter} units")
+        n = {"up": "up", "down": "down"}
+        n.update(names or {})
+        self.names = {k: prefix + v + weight_suffix for k, v in n.items()}
+        self.w_up = self.w_down = self.p_up = self.p_down = None
+
+    def tensors(self) -> Dict[str, TensorDecl]:
+        return {self.names["up"]: TensorDecl((self.inter, self.width), "matrix"),
+                self.names["down"]: TensorDecl((self.width, self.inter), "matrix")}
+
+    def load(self, get: Callable[[str], torch.Tensor], rt: Runtime) -> None:
+        up, down = rt.place(get(self.names["up"]), "matrix"), rt.place(get(self.names["down"]), "matrix")
+        self.p_up, self.p_down = rt.pack(up), rt.pack(down)
+        self.w_up, self.w_down = rt.row_major(up, self.p_up), rt.row_major(down, self.p_down)
+
+    def forward(self, x, ctx=None):
+        rt = self.rt
+        h = linear(rt, x, self.w_up, None, "mlp.up", out_dtype=rt.dtype, packed=self.p_up, act=self.act)
+        return linear(rt, h, self.w_down, None, "mlp.down", packed=self.p_down)

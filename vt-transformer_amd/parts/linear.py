@@ -76,7 +76,7 @@ def takes_prepared_norm(rt: Runtime, n: int, k: int) -> bool:
 
 def linear(rt: Runtime, x: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Tensor], name: str,
            out_dtype: Optional[torch.dtype] = None, bias_lowp: Optional[torch.Tensor] = None,
-           packed=None, residual: Optional[torch.Tensor] = None, hand_on=None):
+           packed=None, residual: Optional[torch.Tensor] = None, hand_on=None, act: Optional[str] = None):
     """x [N, K] in the runtime's dtype -> [N, M].  `name` keys the output's scratch buffer.
     Output dtype: float32 from the hand-written kernels unless `out_dtype` says otherwise; the
     library path returns the 16-bit type (its bias, if any, is `bias_lowp`, the same values in that type).
@@ -85,9 +85,15 @@ def linear(rt: Runtime, x: torch.Tensor, w: torch.Tensor, bias: Optional[torch.T
     its own where that is not possible).  residual (float32 [N, M]): the product is added to it in place and
     `residual` is returned (by the product's kernel where `can_add_residual` says so, else by a kernel after it).
     hand_on (with residual): the norm that comes behind this product (`rms_fusable`); where the kernel can, it
-    prepares that norm on its way and a prepared NormedInput is returned instead of `residual`."""
+    prepares that norm on its way and a prepared NormedInput is returned instead of `residual`.
+    act: an activation on the result (ops.PLAIN_ACTS; without `residual`), by the product's kernel where it is the
+    hand-written 16-bit one, else by a kernel after it."""
+    if act is not None and residual is not None:
+        raise ValueError("an activation on a product that is added to the residual stream")
     n, k = x.shape
     m = w.shape[0] if w is not None else packed.rows * packed.halves   # (no row-major copy: the runtime keeps the packed one only)
+    if act is not None and isinstance(x, NormedInput):
+        x = x.materialize()
     if residual is not None or isinstance(x, NormedInput):
         w_any = packed if packed is not None else w
         is_packed = isinstance(w_any, ops.PackedMatrix)
@@ -121,7 +127,8 @@ def linear(rt: Runtime, x: torch.Tensor, w: torch.Tensor, bias: Optional[torch.T
             return ops.residual_add(residual, linear(rt, x, w, bias, name, out_dtype, bias_lowp, packed))
     if rt.dtype == torch.float32:
         out = rt.buffer(name, (n, m), torch.float32)
-        return ops.linear_f32(x, w, bias, out)
+        ops.linear_f32(x, w, bias, out)
+        return ops.squared_relu(out, out) if act == "squared_relu" else out
     if w is None and not rt.keep_row_major and n >= UNPACK_MIN_ROWS:
         # every product's matrix in turn in the same scratch memory (the largest one's size)
         w = ops.unpack_matrix_bf16(packed, rt.buffer("linear.unpacked", (packed.halves * packed.rows, packed.cols), rt.dtype))
@@ -129,7 +136,7 @@ def linear(rt: Runtime, x: torch.Tensor, w: torch.Tensor, bias: Optional[torch.T
         out = rt.buffer(name, (n, m), out_dtype or torch.float32)
         need = ops.linear_bf16_workspace(n, m, k) if n > 16 else 0
         work = rt.buffer("linear.partials", (need,), torch.float32) if need else None
-        return ops.linear_bf16(x, packed if packed is not None else w, bias, out, work)
+        return ops.linear_bf16(x, packed if packed is not None else w, bias, out, work, act=act)
     out = rt.buffer(name + ".lib", (n, m), rt.dtype)
     if bias is not None:
         if bias_lowp is None:
@@ -137,5 +144,5 @@ def linear(rt: Runtime, x: torch.Tensor, w: torch.Tensor, bias: Optional[torch.T
         torch.addmm(bias_lowp, x, w.t(), out=out)
     else:
         torch.mm(x, w.t(), out=out)
-    return out
+    return ops.squared_relu(out, out) if act == "squared_relu" else out
 

@@ -10,7 +10,7 @@ distance, a learned shift of every score per head, weights that are sigmoids of
 the scores instead of a softmax, neighbouring elements rotated together, a bias
 on the output projection, queries and keys normed over the whole projection
 before it is split into heads, keys and values taken from an earlier layer's
-pages.  Every one of these is a constructor parameter that can be left out.
+pages, a sequence's first keys kept beside a window.  Every one of these is a constructor parameter that can be left out.
 
 Per token: q, k, v (and the gates' logits) in one matrix product with the
 biases; rotation, unit scaling and the write into the pages in one kernel;
@@ -21,6 +21,7 @@ reads the pages; output projection.
     score(i, j) = cap * tanh(scale * q_i . k_j / cap) - slope_h * (i - j)                     (cap 0: scale * q_i . k_j)
     slope_h = 2^(-distance_slopes * (h + 1) / H)                                              (no distance_slopes: 0)
     j is seen from i  <=>  j <= i,  i - j < window (if window > 0),  floor(j / chunk) = floor(i / chunk) (if chunk > 0)
+    keep_first:    j is also seen from i if j <= i and j < keep_first (with a window and no chunks)
     p_ij = exp(score(i, j)) / (sum_j' exp(score(i, j')) + exp(sink_h))                        (no sink: the plain softmax)
     out_i[h] = sigmoid(gate_i[h]) * sum_j p_ij v_j
 
@@ -40,7 +41,7 @@ and scores of its own and writes nothing: its pages are the other layer's, as th
 
 Chunks are counted from position 0 of the sequence.  A key that no later
 position can see is dead for the cache manager: the pages' window is the
-mask's reach.
+mask's reach, and the first keys that a window keeps stay in theirs.
 """
 from __future__ import annotations
 
@@ -77,17 +78,18 @@ def plan_tiles(ctx) -> Optional[Dict[tuple, np.ndarray]]:
 def run_masked_attention(rt: Runtime, ctx, cache, q: torch.Tensor, out: torch.Tensor, nh: int, nkv: int, d: int, dv: int,
                          scale: float, softcap: float = 0.0, window: int = 0, chunk: int = 0, gate=None,
                          gate_column: int = 0, sink=None, slopes=None, dist_log=None, score_shift=None,
-                         sigmoid_weights: bool = False, gate_wide: bool = False) -> torch.Tensor:
+                         sigmoid_weights: bool = False, gate_wide: bool = False, keep_first: int = 0) -> torch.Tensor:
     """The attention itself over a layer's pages, by the kernel that suits the step: in the 16-bit types with heads
     in multiples of 16, steps of single tokens go to the matrix-core kernel whose rows are the heads of a key/value
     group and whose keys are dealt out to many waves, steps with portions of prompts to the one whose rows are tokens
     (tiles planned by `plan_tiles`); everything else, and float32 always, to the kernel with a block per (token, head)."""
     cores = rt.lowp and ops.attention_masked_mfma_takes(d, dv, cache["k"].shape[2])
     kw = dict(gate=gate, gate_column=gate_column, sink=sink, slopes=slopes, dist_log=dist_log, score_shift=score_shift,
-              sigmoid_weights=sigmoid_weights, gate_wide=gate_wide)
+              sigmoid_weights=sigmoid_weights, gate_wide=gate_wide, keep_first=keep_first)
     if cores and ctx.single_token:
         n = q.shape[0]
-        splits = ops.attention_masked_decode_splits(n, nh, nkv, ctx.n_positions, min([w for w in (window, chunk) if w > 0], default=0))
+        splits = ops.attention_masked_decode_splits(n, nh, nkv, ctx.n_positions, min([w for w in (window, chunk) if w > 0], default=0),
+                                                    keep_first)
         part = rt.buffer("mattn.decode_parts", (ops.attention_masked_decode_scratch(n, nh, nkv, dv, splits),), torch.float32)
         return ops.attention_masked_decode(q, cache["k"], cache["v"], ctx.positions, ctx.tok_entry, cache.block_table, out,
                                            part, splits, nh, nkv, d, dv, scale, softcap, window, chunk, **kw)
@@ -116,7 +118,7 @@ class MaskedAttention(Part):
                  q_temp: Optional[Dict[str, float]] = None, value_mix: Optional[str] = None, fuse_norms: bool = False,
                  rot_pairs: str = "halves", qk_gain: bool = False, distance_log: bool = False, score_shift: bool = False,
                  weights: str = "softmax", out_gate: bool = False, o_bias: bool = False,
-                 whole_norm_eps: Optional[float] = None, own_keys: bool = True):
+                 whole_norm_eps: Optional[float] = None, own_keys: bool = True, keep_first: int = 0):
         """key_dim / value_dim: sizes of a head's queries and keys / of its values (default: the same);
         position: a rotary encoding whose `dim` may be smaller than key_dim (the rest of a head passes unchanged);
         unit_rms_eps: queries and keys are divided by their root mean square per head after the rotation, with
@@ -140,7 +142,8 @@ class MaskedAttention(Part):
             whole_norm_eps: queries and keys are divided by the root mean square of the whole projection (eps inside the
             root), tensors q_norm [heads * key_dim] and k_norm [kv heads * key_dim] (None: they are not; without
             rotation, query factor, value mixing and the per-head norm); own_keys False: the layer has no key and value
-            projections (and no k_norm) and reads the cache that its schedule entry names."""
+            projections (and no k_norm) and reads the cache that its schedule entry names; keep_first: how many of a
+            sequence's first keys a window does not pass."""
         if num_heads % num_kv_heads:
             raise ValueError(f"{num_heads} query heads are not a multiple of {num_kv_heads} key/value heads")
         self.rt, self.width = rt, int(width)
@@ -155,6 +158,9 @@ class MaskedAttention(Part):
         self.softcap, self.window, self.chunk = float(softcap), int(window), int(chunk)
         if self.softcap < 0 or self.window < 0 or self.chunk < 0:
             raise ValueError("softcap, window and chunk must not be negative (0 switches each off)")
+        self.keep_first = int(keep_first)
+        if self.keep_first < 0 or (self.keep_first and (not self.window or self.chunk)):
+            raise ValueError(f"keep_first {self.keep_first}: first keys are kept beside a window (and without chunks)")
         self.unit_rms_eps = None if unit_rms_eps is None else float(unit_rms_eps)
         self.has_sink = bool(sink)
         self.distance_slopes = None if not distance_slopes else float(distance_slopes)
@@ -224,7 +230,8 @@ class MaskedAttention(Part):
         chunks, a key is never seen from `chunk` or more positions later."""
         reach = [w for w in (self.window, self.chunk) if w > 0]
         return CacheNeed((PageTensor("k", (self.nkv, self.d), slot_axis=1), PageTensor("v", (self.nkv, self.dv), slot_axis=2)),
-                         window=min(reach) if reach else 0, page_multiple=16 if self._matrix_cores() else 1)
+                         window=min(reach) if reach else 0, page_multiple=16 if self._matrix_cores() else 1,
+                         keep_first=self.keep_first)
 
     def _matrix_cores(self) -> bool:
         """Whether portions of prompts go to the matrix-core kernel: a 16-bit runtime and heads in multiples of 16."""
@@ -351,6 +358,7 @@ class MaskedAttention(Part):
         run_masked_attention(rt, ctx, cache, q, out, nh, nkv, d, dv, self.scale, self.softcap, self.window, self.chunk,
                              gate=y if (self.head_gate or self.out_gate) else None, gate_column=self._gate_column,
                              sink=self.sink, slopes=self.slopes, dist_log=(self.r1, self.r2) if self.distance_log else None,
-                             score_shift=self.shift, sigmoid_weights=self.sigmoid_weights, gate_wide=self.out_gate)
+                             score_shift=self.shift, sigmoid_weights=self.sigmoid_weights, gate_wide=self.out_gate,
+                             keep_first=self.keep_first)
         return linear(rt, out, self.w_o, self.b_o, "mattn.o", bias_lowp=self.b_o_lowp, packed=self.p_o, residual=residual,
                       hand_on=hand_on)

@@ -3,6 +3,10 @@ weighted sum of theirs with two constants,
 
     out = left_scale * left(x) + right_scale * right(x)
 
+or, with `out_norms`, of their results each normed over the model's width,
+
+    out = left_scale * norm_l(left(x)) + right_scale * norm_r(right(x)),    norm(y) = gain * y / sqrt(mean(y^2) + eps)
+
 Either may be any registered mixer.  What they want of the cache manager is
 passed through: pages for at most one of them (a layer has one set of pages),
 and their per-request states one behind the other in one float32 row.
@@ -16,16 +20,23 @@ import torch
 
 from ..config.base import PartSpec
 from ..kernels import ops
-from .base import MIXERS, CacheNeed, Part, Runtime, StateNeed, TensorDecl
+from .base import MIXERS, CacheNeed, Part, Runtime, StateNeed, SublayerPieces, TensorDecl
 
 
 @MIXERS.register("mixer_pair")
 class MixerPair(Part):
     def __init__(self, *, rt: Runtime, width: int, prefix: str, left: PartSpec, right: PartSpec, left_scale: float = 1.0,
-                 right_scale: float = 1.0, shared: Optional[dict] = None):
-        """left, right: the two mixers' specs (a `prefix` among their params stands behind this part's own)."""
+                 right_scale: float = 1.0, out_norms: Optional[dict] = None, shared: Optional[dict] = None):
+        """left, right: the two mixers' specs (a `prefix` among their params stands behind this part's own); out_norms:
+        None, or {eps, left, right}: the eps of the norms on the two results and their gains' tensor names behind the
+        prefix."""
         self.rt, self.width = rt, int(width)
         self.scales = (float(left_scale), float(right_scale))
+        self.norm_eps = float(out_norms["eps"]) if out_norms else None
+        self.norm_names = (prefix + out_norms["left"], prefix + out_norms["right"]) if out_norms else ()
+        self.gains = ()
+        # forward(..., pieces=True): the two results, neither normed nor added up
+        self.hands_pieces = self.norm_eps is not None
         if left.kind == right.kind:
             # (a kind's scratch buffers are keyed by name: the second member would overwrite the first one's result)
             raise ValueError(f"two mixers of one kind ('{left.kind}') side by side are not supported")
@@ -70,13 +81,17 @@ class MixerPair(Part):
         t: Dict[str, TensorDecl] = {}
         for m in self.members:
             t.update(m.tensors())
+        for name in self.norm_names:
+            t[name] = TensorDecl((self.width,), "gain")
         return t
 
     def load(self, get: Callable[[str], torch.Tensor], rt: Runtime) -> None:
         for m in self.members:
             m.load(get, rt)
+        self.gains = tuple(rt.place(get(name), "gain") for name in self.norm_names)
 
-    def forward(self, x, ctx, cache, state):
+    def forward(self, x, ctx, cache, state, pieces: bool = False):
+        """pieces: the result may be returned as SublayerPieces (a pair with norms)."""
         if sum(self.state_floats) and (state is None or state.dim() != 2 or state.shape[1] != sum(self.state_floats)):
             raise RuntimeError("the pair of mixers was given no state of its shape")
         results, at = [], 0
@@ -85,5 +100,10 @@ class MixerPair(Part):
             at += floats
             y = m.forward(x, ctx, cache if m is self.paged else None, own_state)
             results.append(y)
+        if self.norm_eps is not None:
+            (left, right), (gl, gr) = results, self.gains
+            both = SublayerPieces(self.rt, x.shape[0], self.width,
+                                  pair=((left, gl, self.scales[0]), (right, gr, self.scales[1]), self.norm_eps))
+            return both if pieces else both.materialize()
         out = self.rt.buffer("pair.out", tuple(results[0].shape), torch.float32)
         return ops.scaled_sum(results[0], self.scales[0], results[1], self.scales[1], out)

@@ -1,5 +1,5 @@
-"""A feed-forward made of many small gated ones ("experts"), of which a router
-chooses a few for every token.
+"""A feed-forward made of many small ones ("experts", gated or not), of which a
+router chooses a few for every token.
 
     z = W_router x                                  in float32 (the router's matrix is kept in float32)
     s = sigmoid(z)   or   softmax(z)                `score`
@@ -8,6 +8,7 @@ chooses a few for every token.
     weight_on "input":   out = sum_e expert_e(s_e * x)
     weight_on "output":  out = sum_e s_e * expert_e(x)
     expert_e(x) = W_down,e ( f(W_gate,e x) * (W_up,e x) ),   f = SiLU or the tanh form of GELU; no biases
+    expert_e(x) = W_down,e ( max(W_up,e x, 0)^2 )            activation "squared_relu": experts without a gate
 
 Further forms, each a constructor parameter that can be left out:
 
@@ -19,7 +20,7 @@ Further forms, each a constructor parameter that can be left out:
     shared_expert   a feed-forward of any kind that every token runs, added to the experts' sum
 
 The experts' matrices are stacked when they are loaded ([E, 2 F, W] with an expert's gate rows in front of its up rows,
-and [E, W, F]), so a kernel finds an expert by its index.  Nothing of a step's routing reaches the host: the launches
+or [E, F, W] without gates, and [E, W, F]), so a kernel finds an expert by its index.  Nothing of a step's routing reaches the host: the launches
 depend on the number of tokens alone.
 """
 from __future__ import annotations
@@ -44,7 +45,7 @@ class ExpertMixture(Part):
                  renorm_eps: float = 0.0, router_scale: float = 1.0, identity: int = 0, shared_expert: Optional[PartSpec] = None):
         """num_experts experts of intermediate_size, `top` of the router's outputs per token; score, renormalize,
         weight_on, correction, groups {count, keep}, renorm_eps, router_scale, identity: module docstring; activation:
-        "silu" or "gelu_tanh"; shared_expert: a feed-forward whose parameter `prefix` comes behind this part's; names:
+        "silu", "gelu_tanh" or "squared_relu" (no gate; the weight is then on the output); shared_expert: a feed-forward whose parameter `prefix` comes behind this part's; names:
         tensor names behind the prefix for the router, the correction and, with {} standing for an expert's index, for an
         expert's gate, up and down matrices."""
         self.rt, self.width = rt, int(width)
@@ -65,12 +66,15 @@ class ExpertMixture(Part):
             raise ValueError(f"score '{score}' is not known ('sigmoid' and 'softmax' are)")
         if weight_on not in ("input", "output"):
             raise ValueError(f"weight_on '{weight_on}' is not known ('input' and 'output' are)")
-        if activation == "silu":
+        self.gated = activation != "squared_relu"
+        if not self.gated and weight_on != "output":
+            raise ValueError("experts without a gate take their weight on the output")
+        if activation in ("silu", "squared_relu"):
             self.alpha, self.cubic = 1.0, 0.0
         elif activation == "gelu_tanh":
             self.alpha, self.cubic = 2.0 * math.sqrt(2.0 / math.pi), 0.044715      # (1 + tanh z) / 2 = sigmoid(2 z)
         else:
-            raise ValueError(f"activation '{activation}' is not supported ('silu' and 'gelu_tanh' are)")
+            raise ValueError(f"activation '{activation}' is not supported ('silu', 'gelu_tanh' and 'squared_relu' are)")
         self.score, self.renormalize, self.weight_on = score, bool(renormalize), weight_on
         n = {"router": "router", "correction": "correction", "gate": "e{}.gate", "up": "e{}.up", "down": "e{}.down"}
         n.update(names or {})
@@ -95,7 +99,8 @@ class ExpertMixture(Part):
         if self.correction:
             t[nm["correction"]] = TensorDecl((self.n_out,), "bias")
         for e in range(self.ne):
-            t[nm["gate"].format(e)] = TensorDecl((self.inter, self.width), "matrix")
+            if self.gated:
+                t[nm["gate"].format(e)] = TensorDecl((self.inter, self.width), "matrix")
             t[nm["up"].format(e)] = TensorDecl((self.inter, self.width), "matrix")
             t[nm["down"].format(e)] = TensorDecl((self.width, self.inter), "matrix")
         if self.shared is not None:
@@ -109,11 +114,14 @@ class ExpertMixture(Part):
             self.bias = rt.place(get(nm["correction"]), "bias")
         if self.shared is not None:
             self.shared.load(get, rt)
-        self.w_gu = torch.empty((self.ne, 2 * self.inter, self.width), dtype=rt.dtype, device=rt.device)
+        # (w_gu: the first products' matrices, gate rows and up rows, or up rows alone)
+        first = 2 * self.inter if self.gated else self.inter
+        self.w_gu = torch.empty((self.ne, first, self.width), dtype=rt.dtype, device=rt.device)
         self.w_down = torch.empty((self.ne, self.width, self.inter), dtype=rt.dtype, device=rt.device)
         for e in range(self.ne):
-            self.w_gu[e, :self.inter].copy_(rt.place(get(nm["gate"].format(e)), "matrix"))
-            self.w_gu[e, self.inter:].copy_(rt.place(get(nm["up"].format(e)), "matrix"))
+            if self.gated:
+                self.w_gu[e, :self.inter].copy_(rt.place(get(nm["gate"].format(e)), "matrix"))
+            self.w_gu[e, first - self.inter:].copy_(rt.place(get(nm["up"].format(e)), "matrix"))
             self.w_down[e].copy_(rt.place(get(nm["down"].format(e)), "matrix"))
 
     def forward(self, x, ctx=None, pieces: bool = False):
@@ -134,12 +142,18 @@ class ExpertMixture(Part):
         if n * self.top >= self.grouped_from and ops.moe_grouped_ok(x, self.ne, self.width, self.inter):
             plan = rt.buffer("moe.plan", (ops.moe_plan_size(n * self.top, self.ne),), torch.int32)
             ops.moe_sort(ids, plan, self.ne)
-            ops.moe_gate_up_grouped(x, self.w_gu, plan, wts, act, self.top, on_input, self.alpha, self.cubic)
+            if self.gated:
+                ops.moe_gate_up_grouped(x, self.w_gu, plan, wts, act, self.top, on_input, self.alpha, self.cubic)
+            else:
+                ops.moe_up_grouped(x, self.w_gu, plan, act, self.top)
             scratch = rt.buffer("moe.choices", (n * self.top, self.width), torch.float32) if self.top > 1 or not whole else None
             out = rt.buffer("moe.out", (n, self.width), torch.float32) if whole else None
             choices = ops.moe_down_grouped(act, self.w_down, plan, wts, out, scratch, on_output)
         else:
-            ops.moe_gate_up(x, self.w_gu, ids, wts, act, on_input, self.alpha, self.cubic)
+            if self.gated:
+                ops.moe_gate_up(x, self.w_gu, ids, wts, act, on_input, self.alpha, self.cubic)
+            else:
+                ops.moe_up(x, self.w_gu, ids, act)
             # (this kernel adds up a token's choices: one row per token is left)
             choices = ops.moe_down(act, self.w_down, ids, wts, rt.buffer("moe.out", (n, self.width), torch.float32), on_output)
             ids = None

@@ -24,14 +24,16 @@ class RMSNorm(Part):
     rms_fusable = True
 
     def __init__(self, *, rt: Runtime, width: int, prefix: str, eps: float, name: str = "weight", scratch: str = "norm",
-                 unit_offset: bool = False):
-        """unit_offset: the tensor holds w = gain - 1 (the one is added once, in float32, when it is loaded)."""
+                 unit_offset: bool = False, factor: float = 1.0):
+        """unit_offset: the tensor holds w = gain - 1 (the one is added once, in float32, when it is loaded); factor: a
+        constant on the norm's result (the gains are multiplied by it when they are loaded)."""
         self.rt = rt
         self.width = int(width)
         self.eps = float(eps)
         self.name = prefix + name
         self.scratch = scratch
         self.unit_offset = bool(unit_offset)
+        self.factor = float(factor)
         self.gain: Optional[torch.Tensor] = None
 
     def tensors(self) -> Dict[str, TensorDecl]:
@@ -42,6 +44,8 @@ class RMSNorm(Part):
         self.gain = rt.place(get(self.name), "gain")
         if self.unit_offset:
             self.gain = (self.gain + 1.0).contiguous()
+        if self.factor != 1.0:
+            self.gain = (self.gain * self.factor).contiguous()
 
     def forward_streams(self, x: torch.Tensor, w_in: torch.Tensor, rows: Optional[torch.Tensor] = None) -> torch.Tensor:
         """The norm of a weighted sum of several residual streams: x [N, S, H] float32, w_in [S] float32 -> normed
@@ -56,11 +60,14 @@ class RMSNorm(Part):
         out = self.rt.buffer(self.scratch + (".rows" if rows is not None else ""), (n, self.width), self.rt.dtype)
         return ops.rmsnorm(h, delta, self.gain, out, self.eps, rows=rows)
 
-    def forward_output(self, h: torch.Tensor, y, mult: float = 1.0, copy: Optional[torch.Tensor] = None) -> torch.Tensor:
+    def forward_output(self, h: torch.Tensor, y, mult: float = 1.0, copy: Optional[torch.Tensor] = None,
+                       behind: Optional["RMSNorm"] = None) -> torch.Tensor:
         """The norm on a sublayer's output and the addition behind it, in place: h += mult * norm(y).  y [N, H] in any
-        type, or SublayerPieces, which are added up on the way; copy [N, H]: the new h in this tensor's type as well."""
+        type, or SublayerPieces, which are added up on the way; copy [N, H]: the new h in this tensor's type as well, or
+        with `behind` (a norm that is `rms_fusable`) that norm of it."""
         pieces = y.as_args() if isinstance(y, SublayerPieces) else {"y": y}
-        return ops.output_norm_add(h, self.gain, self.eps, mult, copy=copy, **pieces)
+        more = {"next_gain": behind.gain, "next_eps": behind.eps} if behind is not None else {}
+        return ops.output_norm_add(h, self.gain, self.eps, mult, copy=copy, **pieces, **more)
 
 
 @NORMS.register("layernorm")

@@ -40,13 +40,30 @@ def stretched_frequencies(inv: np.ndarray, dims: int, theta: float, factor: floa
     return inv / factor * ramp + inv * (1.0 - ramp), 0.1 * math.log(factor) + 1.0
 
 
+def banded_frequencies(inv: np.ndarray, factor: float, original: float, low: float, high: float) -> np.ndarray:
+    """Frequencies for contexts `factor` times longer than the `original` one, by bands of how often a pair turns within
+    it (original / wavelength; the scheme of Llama 3.1): one that turns more than `high` times keeps its frequency, one
+    that turns fewer than `low` times is slowed down by `factor`, and between the two both are mixed, linearly in the
+    number of turns."""
+    turns = original * inv / (2.0 * math.pi)
+    share = np.clip((turns - low) / max(high - low, 1e-300), 0.0, 1.0)
+    return share * inv + (1.0 - share) * inv / factor
+
+
+# kinds of scaling: the constants that each takes
+SCALINGS = {"ramp": ("factor", "original", "fast", "slow"), "bands": ("factor", "original", "low", "high")}
+
+
 def rotary_table(n_positions: int, dims: int, theta: float, scaling: Optional[dict] = None) -> Tuple[np.ndarray, np.ndarray]:
-    """(cos, sin), float32 [n_positions, dims/2].  scaling: None, or the constants of `stretched_frequencies`
-    (factor, original, fast, slow)."""
+    """(cos, sin), float32 [n_positions, dims/2].  scaling: None, or a kind (absent: "ramp") with its constants:
+    "ramp" those of `stretched_frequencies` (factor, original, fast, slow), "bands" those of `banded_frequencies` (factor,
+    original, low, high)."""
     i = np.arange(0, dims, 2, dtype=np.float64)
     inv = 1.0 / np.power(np.float64(theta), i / dims)
     mag = 1.0
-    if scaling:
+    if scaling and scaling.get("kind", "ramp") == "bands":
+        inv = banded_frequencies(inv, float(scaling["factor"]), float(scaling["original"]), float(scaling["low"]), float(scaling["high"]))
+    elif scaling:
         inv, mag = stretched_frequencies(inv, dims, theta, float(scaling["factor"]), float(scaling["original"]),
                                          float(scaling["fast"]), float(scaling["slow"]))
     ang = np.arange(n_positions, dtype=np.float64)[:, None] * inv[None, :]
@@ -59,7 +76,7 @@ class RotaryEncoding(Part):
 
     def __init__(self, *, rt: Runtime, theta: float, dim: int, scaling: Optional[dict] = None):
         """dim: how many of a head's leading elements are rotated (the rest pass unchanged where the mixer's head is
-        larger); scaling: None or {factor, original, fast, slow} (`stretched_frequencies`)."""
+        larger); scaling: None or {kind, and the constants that the kind takes} (`rotary_table`)."""
         if dim % 2 or dim <= 0:
             raise ValueError(f"rotary dims {dim} must be even and positive")
         self.rt = rt
@@ -67,7 +84,10 @@ class RotaryEncoding(Part):
         self.dim = int(dim)
         self.scaling = dict(scaling) if scaling else None
         if self.scaling:
-            for key in ("factor", "original", "fast", "slow"):
+            kind = self.scaling.get("kind", "ramp")
+            if kind not in SCALINGS:
+                raise ValueError(f"rotary scaling '{kind}' is not known ({', '.join(SCALINGS)})")
+            for key in SCALINGS[kind]:
                 if key not in self.scaling or not float(self.scaling[key]) > 0:
                     raise ValueError(f"rotary scaling needs a positive '{key}'")
         self._tables: Optional[Tuple[torch.Tensor, torch.Tensor]] = None
