@@ -274,6 +274,26 @@ def tipetar_pair_configs(key: str, window: int):
     return tip, kig
 
 
+def lilatar_pair_configs(key: str, window: int):
+    """(Lilatar config.json, Fedovik config.json) of equal sizes.  Lilatar: the pair of attention (capped, over `window`
+    positions and the first 64) and channel-decay delta rule in turn with linear attention of a constant decay, all with
+    the same heads; behind them two dense feed-forwards and two mixtures of sixteen experts (four a token, an eighth of
+    the dense size each) in turn.  Fedovik: the pair of `fedovik_pair_configs`."""
+    width, layers, heads, kv, d, ff, vocab = PAIR_SIZES[key]
+    dense = {"kind": "dense", "ff": ff}
+    moe = {"kind": "moe", "expert": {"ff": ff // 8}, "router": {"experts": 16, "top": 4}}
+    pair = {"left": {"heads": heads, "kv_heads": kv, "dim": d, "vdim": d, "scale": d ** -0.5, "softcap": 30.0,
+                     "mask": {"size": window, "keep_first": 64},
+                     "rot": {"dims": d // 2, "base": 5e5, "scaling": {"factor": 8.0, "original": 8192, "low": 1.0, "high": 4.0}}},
+            "right": {"heads": heads, "kv_heads": kv, "dim": d, "vdim": d, "conv": 4, "a_rank": 64, "g_rank": 64}}
+    lin = {"heads": heads, "dim": d, "vdim": d, "decay": [1.0 - 2.0 ** (-1.0 - 7.0 * h / max(heads - 1, 1)) for h in range(heads)]}
+    lil = {"architecture": "Lilatar", "vocab": vocab, "width": width, "norm": {"eps": 1e-6}, "logit_scale": 0.5,
+           "layers": [{"type": "parallel" if i % 2 == 0 else "lightning", "mixer": pair if i % 2 == 0 else lin,
+                       "mlp": dense if i % 4 < 2 else moe} for i in range(layers)], "max_positions": 32768}
+    fed, _ = fedovik_pair_configs(key, window)
+    return lil, fed
+
+
 class PairBench(Bench):
     """Bench's measurements on an engine built from any config.json."""
 
@@ -297,9 +317,9 @@ class PairBench(Bench):
 
 def design_pairs(args, design: str) -> int:
     """Prefill and decode of a second design (lisunex or gabelorn beside Qwen2, kigalix beside Gabelorn, fedovik beside
-    Lisunex, tipetar beside Kigalix) at equal sizes; one JSON line."""
+    Lisunex, tipetar beside Kigalix, lilatar beside Fedovik) at equal sizes; one JSON line."""
     title = design.capitalize()
-    beside = {"kigalix": "gabelorn", "fedovik": "lisunex", "tipetar": "kigalix"}.get(design, "qwen2")
+    beside = {"kigalix": "gabelorn", "fedovik": "lisunex", "tipetar": "kigalix", "lilatar": "fedovik"}.get(design, "qwen2")
     keys = [k.strip() for k in getattr(args, design).split(",") if k.strip()]
     for k in keys:
         if k not in PAIR_SIZES:
@@ -309,9 +329,11 @@ def design_pairs(args, design: str) -> int:
     per_req = -(-(prompt_len + args.steps + args.warmup + 32) // 16) * 16
     pool = max(batch * per_req, T + 64)
     span = {"lisunex": args.lisunex_chunk, "gabelorn": args.gabelorn_window, "kigalix": args.kigalix_streams,
-            "fedovik": args.fedovik_window, "tipetar": args.tipetar_window}[design]
+            "fedovik": args.fedovik_window, "tipetar": args.tipetar_window,
+            "lilatar": args.lilatar_window}[design]
     make = {"lisunex": pair_configs, "gabelorn": gabelorn_pair_configs, "kigalix": kigalix_pair_configs,
-            "fedovik": fedovik_pair_configs, "tipetar": tipetar_pair_configs}[design]
+            "fedovik": fedovik_pair_configs, "tipetar": tipetar_pair_configs,
+            "lilatar": lilatar_pair_configs}[design]
     only = getattr(args, "only", "")
     out = {}
     for k in keys:
@@ -344,7 +366,7 @@ def design_pairs(args, design: str) -> int:
         "data": "synthetic (random weights N(0,0.02), uniform random token ids)",
         "config": {"model": f"{title} and {beside.capitalize()} at equal sizes", "global_batch": batch, "seq_len": prompt_len,
                    "prefill_tokens": T, {"lisunex": "chunk", "gabelorn": "window", "kigalix": "streams", "fedovik": "window",
-                                          "tipetar": "window"}[design]: span,
+                                          "tipetar": "window", "lilatar": "window"}[design]: span,
                    "parallelism": "1 GPU"},
         "pairs": out}), flush=True)
     return 0
@@ -416,15 +438,21 @@ def main() -> int:
                          "(latent attention and as many experts) at equal sizes, prefill of --prefill-tokens and decode at "
                          "--batch; sizes by name, with commas: " + ", ".join(PAIR_SIZES))
     ap.add_argument("--tipetar-window", type=int, default=1024, help="positions that a Tipetar layer sees")
+    ap.add_argument("--lilatar", default="", metavar="SIZES",
+                    help="another workload instead: the Lilatar design (windowed attention beside a channel-decay delta rule in "
+                         "turn with linear attention, dense and expert feed-forwards of squared ReLU) beside Fedovik at equal "
+                         "sizes, prefill of --prefill-tokens and decode at --batch; sizes by name, with commas: " + ", ".join(PAIR_SIZES))
+    ap.add_argument("--lilatar-window", type=int, default=1024, help="positions that the windowed attention of Lilatar (and of "
+                    "Fedovik beside it) sees; Lilatar's sees the first 64 as well")
     ap.add_argument("--only", default="", metavar="MODEL",
-                    help="with --lisunex, --gabelorn, --kigalix, --fedovik or --tipetar: measure one model of the pair alone "
+                    help="with --lisunex, --gabelorn, --kigalix, --fedovik, --tipetar or --lilatar: measure one model of the pair alone "
                          "(profiling runs)")
     args = ap.parse_args()
     if args.gpus != 1 or int(os.environ.get("WORLD_SIZE", "1")) != 1:
         print("bench.py: this engine runs on one GPU; N > 1 is not measured")
         return 2
 
-    designs = [d for d in ("lisunex", "gabelorn", "kigalix", "fedovik", "tipetar") if getattr(args, d)]
+    designs = [d for d in ("lisunex", "gabelorn", "kigalix", "fedovik", "tipetar", "lilatar") if getattr(args, d)]
     if designs:
         if args.dtype == "float16":
             args.dtype = "bfloat16"         # the serving dtype of these designs

@@ -1455,6 +1455,43 @@ def decayed_attention(x: torch.Tensor, q_column: int, k_column: int, v_column: i
     return out
 
 
+DECAYED_CHUNK = 64      # tokens of a chunk of decayed_attention_chunked
+
+
+def decayed_attention_chunks_take(key_dim: int, value_dim: int) -> bool:
+    """Whether decayed_attention_chunked takes heads of these sizes."""
+    return key_dim % 4 == 0 and value_dim % 4 == 0 and key_dim <= DELTA_MAX_KEY_DIM
+
+
+def decayed_attention_chunked(x: torch.Tensor, q_column: int, k_column: int, v_column: int, powers: torch.Tensor, state: torch.Tensor,
+                              plan: torch.Tensor, n_chunks: int, slots: torch.Tensor, work: torch.Tensor, out: torch.Tensor,
+                              n_heads: int, key_dim: int, value_dim: int, silu: bool = True) -> torch.Tensor:
+    """decayed_attention for portions of prompts, on the matrix cores in float32.  powers (float32 [H, DECAYED_CHUNK + 1]):
+    every head's decay to the powers 0, 1, ..; plan (int32): where every entry's chunks start (entries + 1 numbers), then
+    per chunk its first row and its rows, runs of at most DECAYED_CHUNK tokens of one entry in order; work: float32 scratch of
+    n_chunks * H * Dv * D."""
+    n = x.shape[0]
+    hd = n_heads * key_dim
+    _chk(x, "decayed_attention_chunked.x")
+    if x.dim() != 2 or min(q_column, k_column, v_column) < 0 or \
+            x.shape[1] < max(max(q_column, k_column) + hd, v_column + n_heads * value_dim):
+        raise KernelError(f"decayed_attention_chunked.x: shape {tuple(x.shape)} does not hold its columns")
+    if not decayed_attention_chunks_take(key_dim, value_dim):
+        raise KernelError(f"decayed_attention_chunked: heads of {key_dim}/{value_dim} (multiples of 4, keys up to {DELTA_MAX_KEY_DIM})")
+    entries = slots.numel()
+    _chk(powers, "decayed_attention_chunked.powers", torch.float32, (n_heads, DECAYED_CHUNK + 1))
+    _chk(out, "decayed_attention_chunked.out", torch.float32, (n, n_heads * value_dim))
+    _chk(plan, "decayed_attention_chunked.plan", torch.int32, (entries + 1 + 2 * n_chunks,))
+    _chk(slots, "decayed_attention_chunked.slots", torch.int32)
+    _chk(work, "decayed_attention_chunked.work", torch.float32)
+    sp, ss = _state_rows(state, "decayed_attention_chunked", n_heads * key_dim * value_dim)
+    _run(load_lib("vt_linear_attn", half=_half(x)), "vt_decayed_attn_chunked", _ptr(x), _i(_code(x)), ctypes.c_longlong(x.stride(0)),
+         _i(q_column), _i(k_column), _i(v_column), _ptr(powers), sp, ss, _ptr(plan), _ptr(slots), _ptr(work),
+         ctypes.c_longlong(work.numel()), _ptr(out), _i(entries), _i(n_chunks), _i(n_heads), _i(key_dim), _i(value_dim),
+         _i(1 if silu else 0), _stream())
+    return out
+
+
 # ---------------------------------------------------------------------------
 # several residual streams and the token shift (vt_streams.hip)
 STREAMS_MAX = 8
