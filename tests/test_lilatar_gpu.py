@@ -398,15 +398,18 @@ def test_experts_without_a_gate(dtype, experts, top, inter, width):
         assert isinstance(pieces, SublayerPieces) and rel(pieces.materialize(), got) < 1e-6
 
 
-@pytest.mark.parametrize("heads,dim", [(1, 40), (3, 200), (1, 513), (1, 2048), (2, 700)])
+@pytest.mark.parametrize("heads,dim", [(1, 40), (3, 200), (1, 513), (1, 900), (1, 2048), (2, 700), (1, 3000), (1, 4100)])
 def test_gated_norm_over_wide_heads(heads, dim):
     from vt_transformer_amd.kernels import ops
     g = torch.Generator().manual_seed(dim)
     o, gate, w = torch.randn(6, heads * dim, generator=g), torch.randn(6, heads * dim + 8, generator=g), torch.randn(heads * dim, generator=g)
-    out = torch.empty(6, heads * dim, device=DEV)
-    ops.gated_rmsnorm(o.to(DEV), w.to(DEV), gate.to(DEV), 5, out, heads, dim, 1e-3, gate_kind="sigmoid")
-    ref = pl.unit_rms(o.double().reshape(6, heads, dim), 1e-3).reshape(6, -1) * w.double() * torch.sigmoid(gate.double()[:, 5:5 + heads * dim])
-    assert rel(out, ref) < 3e-6
+    for column in (4, 5):       # (16-byte accesses, and not)
+        for gdt, odt in ((torch.float32, torch.float32), (torch.float32, torch.bfloat16), (torch.bfloat16, torch.bfloat16)):
+            gd, out = gate.to(gdt), torch.empty(6, heads * dim, dtype=odt, device=DEV)
+            for kind, f in (("sigmoid", torch.sigmoid), ("silu", pl.silu)):
+                ops.gated_rmsnorm(o.to(DEV), w.to(DEV), gd.to(DEV), column, out, heads, dim, 1e-3, gate_kind=kind)
+                ref = pl.unit_rms(o.double().reshape(6, heads, dim), 1e-3).reshape(6, -1) * w.double() * f(gd.double()[:, column:column + heads * dim])
+                assert rel(out, ref) < (3e-6 if odt == torch.float32 else 6e-3)
 
 
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])

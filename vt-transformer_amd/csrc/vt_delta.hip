@@ -391,6 +391,51 @@ __global__ __launch_bounds__(THREADS) void gated_rmsnorm_kernel(const float* __r
     }
 }
 
+// Wide heads of a multiple of 4 elements up to 1024 NV: a thread keeps NV pieces of four in registers between the sum of
+// squares and the scaling, and weights and gates are asked for in front of the sum.
+__device__ __forceinline__ float4 gn_load4(const float* p) { return *(const float4*)p; }
+__device__ __forceinline__ float4 gn_load4(const bf16_t* p) {
+    const uint2 u = *(const uint2*)p;
+    return make_float4(lowp_lo(u.x), lowp_hi(u.x), lowp_lo(u.y), lowp_hi(u.y));
+}
+__device__ __forceinline__ void gn_store4(float* p, float4 v) { *(float4*)p = v; }
+__device__ __forceinline__ void gn_store4(bf16_t* p, float4 v) { *(uint2*)p = make_uint2(vt_pack2(v.x, v.y), vt_pack2(v.z, v.w)); }
+template <typename TG, typename TO, int NV>
+__global__ __launch_bounds__(256) void gated_rmsnorm_vec_kernel(const float* __restrict__ o, const float* __restrict__ w,
+                                                                const TG* __restrict__ gate, long long ldg, TO* __restrict__ out,
+                                                                int H, int Dv, float eps, int w_stride, int gate_kind) {
+    __shared__ float red[16];
+    const int t = blockIdx.x, h = blockIdx.y, n4 = Dv >> 2;
+    const float* row = o + ((size_t)t * H + h) * Dv;
+    const float* wh = w + (size_t)h * w_stride;
+    const TG* gr = gate + (size_t)t * ldg + (size_t)h * Dv;
+    TO* dst = out + ((size_t)t * H + h) * Dv;
+    float4 v[NV], wv[NV], gv[NV];
+    float ss = 0.f;
+#pragma unroll
+    for (int i = 0; i < NV; ++i) {
+        const int q = threadIdx.x + 256 * i;
+        v[i] = make_float4(0.f, 0.f, 0.f, 0.f);
+        if (q < n4) {
+            v[i] = gn_load4(row + 4 * q);
+            wv[i] = gn_load4(wh + 4 * q);
+            gv[i] = gn_load4(gr + 4 * q);
+        }
+    }
+#pragma unroll
+    for (int i = 0; i < NV; ++i) ss = fmaf(v[i].x, v[i].x, fmaf(v[i].y, v[i].y, fmaf(v[i].z, v[i].z, fmaf(v[i].w, v[i].w, ss))));
+    ss = block_sum(ss, red);
+    const float rinv = 1.0f / sqrtf(ss / (float)Dv + eps);
+    auto act = [&](float z) { return gate_kind ? 1.0f / (1.0f + expf(-z)) : silu_f(z); };
+#pragma unroll
+    for (int i = 0; i < NV; ++i) {
+        const int q = threadIdx.x + 256 * i;
+        if (q < n4)
+            gn_store4(dst + 4 * q, make_float4(v[i].x * rinv * wv[i].x * act(gv[i].x), v[i].y * rinv * wv[i].y * act(gv[i].y),
+                                               v[i].z * rinv * wv[i].z * act(gv[i].z), v[i].w * rinv * wv[i].w * act(gv[i].w)));
+    }
+}
+
 extern "C" int vt_gated_rmsnorm(const float* o, const float* w, const void* gate, int gate_dtype, long long ldg, void* out,
                                 int out_dtype, int n, int H, int Dv, float eps, int w_per_head, int gate_kind,
                                 hipStream_t stream) {
@@ -400,14 +445,21 @@ extern "C" int vt_gated_rmsnorm(const float* o, const float* w, const void* gate
     if (n == 0) return 0;
     const dim3 grid(n, H);
     const int ws = w_per_head ? Dv : 0;
+    const bool vec = Dv > 512 && Dv <= 4096 && Dv % 4 == 0 && ldg % 4 == 0 &&
+                     !(((uintptr_t)o | (uintptr_t)w | (uintptr_t)gate | (uintptr_t)out) & 15);
+#define VT_GNORM_VEC(TG, TO, NV) gated_rmsnorm_vec_kernel<TG, TO, NV><<<grid, 256, 0, stream>>>(o, w, (const TG*)gate, ldg, (TO*)out, H, Dv, eps, ws, gate_kind)
 #define VT_GNORM(TG, TO) do { \
-        if (Dv > 512) gated_rmsnorm_kernel<TG, TO, 256><<<grid, 256, 0, stream>>>(o, w, (const TG*)gate, ldg, (TO*)out, H, Dv, eps, ws, gate_kind); \
+        if (vec && Dv <= 1024) VT_GNORM_VEC(TG, TO, 1); \
+        else if (vec && Dv <= 2048) VT_GNORM_VEC(TG, TO, 2); \
+        else if (vec) VT_GNORM_VEC(TG, TO, 4); \
+        else if (Dv > 512) gated_rmsnorm_kernel<TG, TO, 256><<<grid, 256, 0, stream>>>(o, w, (const TG*)gate, ldg, (TO*)out, H, Dv, eps, ws, gate_kind); \
         else gated_rmsnorm_kernel<TG, TO, 64><<<grid, 64, 0, stream>>>(o, w, (const TG*)gate, ldg, (TO*)out, H, Dv, eps, ws, gate_kind); } while (0)
     if (gate_dtype == VT_F32 && out_dtype == VT_F32) VT_GNORM(float, float);
     else if (gate_dtype == VT_F32 && out_dtype == VT_BF16) VT_GNORM(float, bf16_t);
     else if (gate_dtype == VT_BF16 && out_dtype == VT_BF16) VT_GNORM(bf16_t, bf16_t);
     else return vt_fail("vt_gated_rmsnorm: dtypes %d -> %d are not handled", gate_dtype, out_dtype);
 #undef VT_GNORM
+#undef VT_GNORM_VEC
     VT_CHECK_LAUNCH("vt_gated_rmsnorm");
     return 0;
 }

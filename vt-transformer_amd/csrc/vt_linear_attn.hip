@@ -52,8 +52,18 @@ struct DecayedArgs {
     int H, D, Dv, silu;
 };
 
-// One token per entry: entry e's is token e.
-template <typename TI, int DS>
+__device__ __forceinline__ void read4(const float* p, float* v) {
+    const float4 f = *(const float4*)p;
+    v[0] = f.x; v[1] = f.y; v[2] = f.z; v[3] = f.w;
+}
+__device__ __forceinline__ void read4(const bf16_t* p, float* v) {
+    const uint2 u = *(const uint2*)p;
+    v[0] = lowp_lo(u.x); v[1] = lowp_hi(u.x); v[2] = lowp_lo(u.y); v[3] = lowp_hi(u.y);
+}
+
+// One token per entry: entry e's is token e.  VEC: keys of a multiple of 4 elements that lie at multiples of 4 (a lane's
+// groups of four are then 16-byte accesses, whole or not at all).
+template <typename TI, int DS, bool VEC>
 __global__ __launch_bounds__(256) void decayed_step_kernel(DecayedArgs a) {
     const int e = blockIdx.x, h = blockIdx.y;
     const int tid = threadIdx.x, r = tid & 15;
@@ -63,13 +73,27 @@ __global__ __launch_bounds__(256) void decayed_step_kernel(DecayedArgs a) {
     float* S = a.state + (size_t)a.slots[e] * a.slot_stride + ((size_t)h * Dv + col) * D;
     if (col >= Dv) return;      // (a row of lanes leaves together)
     float s[DS], k[DS], q[DS];
+    if constexpr (VEC) {
 #pragma unroll
-    for (int i = 0; i < DS; ++i) {
-        const int d = lane_elem<DS>(r, i);
-        const bool in = d < D;
-        s[i] = in ? S[d] : 0.f;
-        k[i] = in ? load_f32<TI>(x, a.k_col + (size_t)h * D + d) : 0.f;
-        q[i] = in ? load_f32<TI>(x, a.q_col + (size_t)h * D + d) : 0.f;
+        for (int i = 0; i < DS; i += 4) {
+            const int d = lane_elem<DS>(r, i);
+#pragma unroll
+            for (int j = 0; j < 4; ++j) s[i + j] = k[i + j] = q[i + j] = 0.f;
+            if (d < D) {
+                read4(S + d, s + i);
+                read4(x + a.k_col + (size_t)h * D + d, k + i);
+                read4(x + a.q_col + (size_t)h * D + d, q + i);
+            }
+        }
+    } else {
+#pragma unroll
+        for (int i = 0; i < DS; ++i) {
+            const int d = lane_elem<DS>(r, i);
+            const bool in = d < D;
+            s[i] = in ? S[d] : 0.f;
+            k[i] = in ? load_f32<TI>(x, a.k_col + (size_t)h * D + d) : 0.f;
+            q[i] = in ? load_f32<TI>(x, a.q_col + (size_t)h * D + d) : 0.f;
+        }
     }
     float v = load_f32<TI>(x, a.v_col + (size_t)h * Dv + col);
     const float g = a.decay[h];
@@ -83,8 +107,19 @@ __global__ __launch_bounds__(256) void decayed_step_kernel(DecayedArgs a) {
         }
         s[i] = fmaf(g, s[i], k[i] * v);
         acc = fmaf(q[i], s[i], acc);
-        const int d = lane_elem<DS>(r, i);
-        if (d < D) S[d] = s[i];
+    }
+    if constexpr (VEC) {
+#pragma unroll
+        for (int i = 0; i < DS; i += 4) {
+            const int d = lane_elem<DS>(r, i);
+            if (d < D) *(float4*)(S + d) = make_float4(s[i], s[i + 1], s[i + 2], s[i + 3]);
+        }
+    } else {
+#pragma unroll
+        for (int i = 0; i < DS; ++i) {
+            const int d = lane_elem<DS>(r, i);
+            if (d < D) S[d] = s[i];
+        }
     }
     acc = row16_sum(acc);
     if (r == 0) a.o[((size_t)e * a.H + h) * Dv + col] = acc;
@@ -184,23 +219,36 @@ extern "C" int vt_decayed_attn(const void* x, int dtype, long long ldx, int q_co
     a.slot_stride = slot_stride; a.q_col = q_col; a.k_col = k_col; a.v_col = v_col; a.H = H; a.D = D; a.Dv = Dv; a.silu = silu;
     const int share = (D + 15) / 16;
     const dim3 grid(n_entries, H, (Dv + ROWS - 1) / ROWS);
-#define VT_DECAYED_DS(KERNEL, TI)                                                            \
+    const bool vec = D % 4 == 0 && !((slot_stride | ldx | q_col | k_col) & 3) && !(((uintptr_t)state | (uintptr_t)x) & 15);
+#define VT_DECAYED_STEP(TI)                                                                  \
     do {                                                                                     \
-        if (share <= 1) KERNEL<TI, 1><<<grid, 256, 0, stream>>>(a);                          \
-        else if (share <= 2) KERNEL<TI, 2><<<grid, 256, 0, stream>>>(a);                     \
-        else if (share <= 4) KERNEL<TI, 4><<<grid, 256, 0, stream>>>(a);                     \
-        else if (share <= 8) KERNEL<TI, 8><<<grid, 256, 0, stream>>>(a);                     \
-        else KERNEL<TI, 16><<<grid, 256, 0, stream>>>(a);                                    \
+        if (share <= 1) decayed_step_kernel<TI, 1, false><<<grid, 256, 0, stream>>>(a);      \
+        else if (share <= 2) decayed_step_kernel<TI, 2, false><<<grid, 256, 0, stream>>>(a); \
+        else if (share <= 4 && vec) decayed_step_kernel<TI, 4, true><<<grid, 256, 0, stream>>>(a);   \
+        else if (share <= 4) decayed_step_kernel<TI, 4, false><<<grid, 256, 0, stream>>>(a);         \
+        else if (share <= 8 && vec) decayed_step_kernel<TI, 8, true><<<grid, 256, 0, stream>>>(a);   \
+        else if (share <= 8) decayed_step_kernel<TI, 8, false><<<grid, 256, 0, stream>>>(a);         \
+        else if (vec) decayed_step_kernel<TI, 16, true><<<grid, 256, 0, stream>>>(a);        \
+        else decayed_step_kernel<TI, 16, false><<<grid, 256, 0, stream>>>(a);                \
+    } while (0)
+#define VT_DECAYED_SCAN(TI)                                                                  \
+    do {                                                                                     \
+        if (share <= 1) decayed_scan_kernel<TI, 1><<<grid, 256, 0, stream>>>(a);             \
+        else if (share <= 2) decayed_scan_kernel<TI, 2><<<grid, 256, 0, stream>>>(a);        \
+        else if (share <= 4) decayed_scan_kernel<TI, 4><<<grid, 256, 0, stream>>>(a);        \
+        else if (share <= 8) decayed_scan_kernel<TI, 8><<<grid, 256, 0, stream>>>(a);        \
+        else decayed_scan_kernel<TI, 16><<<grid, 256, 0, stream>>>(a);                       \
     } while (0)
     if (dtype != VT_F32 && dtype != VT_BF16) return vt_fail("vt_decayed_attn: unknown dtype %d", dtype);
     if (single) {
-        if (dtype == VT_F32) VT_DECAYED_DS(decayed_step_kernel, float);
-        else VT_DECAYED_DS(decayed_step_kernel, bf16_t);
+        if (dtype == VT_F32) VT_DECAYED_STEP(float);
+        else VT_DECAYED_STEP(bf16_t);
     } else {
-        if (dtype == VT_F32) VT_DECAYED_DS(decayed_scan_kernel, float);
-        else VT_DECAYED_DS(decayed_scan_kernel, bf16_t);
+        if (dtype == VT_F32) VT_DECAYED_SCAN(float);
+        else VT_DECAYED_SCAN(bf16_t);
     }
-#undef VT_DECAYED_DS
+#undef VT_DECAYED_STEP
+#undef VT_DECAYED_SCAN
     VT_CHECK_LAUNCH("vt_decayed_attn");
     return 0;
 }
